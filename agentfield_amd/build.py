@@ -45,22 +45,27 @@ HIP_SOURCES = [
 #           residual, norms, gated units, routers)
 #   seq     masked softmax attention + decayed linear recurrences
 #   ssm     selective state-space scan + sigmoid attention
-#   hyper   multi-stream residual mixing, input convolutions, latent-attention
-#           row steps
+#   hyper   multi-stream residual mixing, input convolutions
+#   latent  latent-attention row steps, gated head outputs
+#   rope    rotary tables, per-head q/k norm with rotary positions, page append
 #   conv    short depthwise causal convolution with carried inputs
-#   delta   gated delta-rule recurrence, per-head q/k norm with rotary
-#           positions, norm after the residual sum
+#   delta   gated delta-rule recurrence, norm after the residual sum
+#   rglru   real-gated linear recurrent unit
 MIX_GROUPS = {
     "glue": (PKG_DIR / "libafglue.so", ["mix_glue.hip"]),
     "seq": (PKG_DIR / "libafmix.so", ["mix_seq.hip", "mix_attn_mfma.hip"]),
     "ssm": (PKG_DIR / "libafssm.so", ["mix_ssm.hip", "mix_sigattn.hip",
                                        "mix_sigattn_mfma.hip"]),
     "hyper": (PKG_DIR / "libafhyper.so", ["mix_hyper.hip"]),
+    "latent": (PKG_DIR / "libaflatent.so", ["mix_latent.hip"]),
+    "rope": (PKG_DIR / "libafrope.so", ["mix_rope.hip"]),
     "delta": (PKG_DIR / "libafdelta.so", ["mix_delta.hip"]),
     "conv": (PKG_DIR / "libafconv.so", ["mix_conv.hip"]),
+    "rglru": (PKG_DIR / "libafrglru.so", ["mix_rglru.hip"]),
 }
 MIX_SOURCES = [s for _lib, srcs in MIX_GROUPS.values() for s in srcs]
 MIX_LIB = MIX_GROUPS["seq"][0]
+HEADERS = ["common.h", "mix_attn.h", "mix_rows.h"]
 
 # hipcc -O3 may otherwise fuse scalar float code into packed-fp32 VALU ops
 HIP_FLAGS = ["-O3", "-std=c++17", "-fPIC", "-fvisibility=hidden",
@@ -72,7 +77,7 @@ def _needs_build(lib: Path = LIB, sources=None) -> bool:
         return True
     lib_m = lib.stat().st_mtime
     deps = [CSRC / s for s in (sources or HIP_SOURCES)] + \
-        [CSRC / "common.h", CSRC / "mix_attn.h", Path(__file__)]
+        [CSRC / h for h in HEADERS] + [Path(__file__)]
     return any(d.stat().st_mtime > lib_m for d in deps)
 
 
@@ -117,7 +122,8 @@ def _build_lib(lib: Path, sources, force: bool, verbose: bool) -> Path:
         objs.append(op)
         if (not force and op.exists()
                 and op.stat().st_mtime > sp.stat().st_mtime
-                and op.stat().st_mtime > (CSRC / "common.h").stat().st_mtime):
+                and all(op.stat().st_mtime > (CSRC / h).stat().st_mtime
+                        for h in HEADERS)):
             continue
         cmd = [
             HIPCC, f"--offload-arch={ARCH}", *HIP_FLAGS,

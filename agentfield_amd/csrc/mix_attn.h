@@ -13,6 +13,10 @@
 // ldv is the row stride of the value pages in elements: dv for pages of
 // their own, dk when the values are the leading dv elements of the key rows
 // (vc == kc; latent attention keeps one row per token).
+//
+// vshare > 1: the value pages have G / vshare heads, each serving vshare
+// neighbouring key heads (differential attention: the two maps of a K/V head
+// have keys of their own over the same values).
 #pragma once
 #include "common.h"
 
@@ -23,6 +27,7 @@ struct AttnExtra {
   float cap;           // 0: no soft cap
   i64 ldv;
   int first;           // 0: no always-visible leading keys
+  int vshare;          // key heads per value head
 };
 
 // exact forms (fp32 storage and the row kernels)

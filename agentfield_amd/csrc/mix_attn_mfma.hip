@@ -49,31 +49,37 @@ __device__ __forceinline__ s16x8 load8(const u16* row, int e0, int n) {
 // Stage one tile of KT keys: K rows row-major into k_lds, V rows transposed into
 // v_lds ([d][token], token pairs packed into 32-bit writes).  The page walk
 // is done once per key (row_lds[tok] = row index in the pages, -1 for keys
-// past `last`), so the tile's loads depend on nothing but LDS and are issued
-// back to back.
-template <int DKC, int DVT, bool VEC, int NT = 256, int KT = 64>
+// past `last`; vrow_lds the value row, whose pages may have fewer heads), so
+// the tile's loads depend on nothing but LDS and are issued back to back.
+// NK = 2 stages the rows of the key heads g and g + 1, one tile behind the
+// other, over one value tile.
+template <int DKC, int DVT, bool VEC, int NT = 256, int KT = 64, int NK = 1>
 __device__ __forceinline__ void stage_kv_tile(
-    u16* k_lds, u16* v_lds, i32* row_lds, const u16* __restrict__ kc,
-    const u16* __restrict__ vc, const i32* __restrict__ btr, int kv0, int last,
-    int G, int g, int page, int dk, int dv, i64 ldv) {
+    u16* k_lds, u16* v_lds, i32* row_lds, i32* vrow_lds,
+    const u16* __restrict__ kc, const u16* __restrict__ vc,
+    const i32* __restrict__ btr, int kv0, int last, int G, int g, int GV,
+    int gv, int page, int dk, int dv, i64 ldv) {
   constexpr int KS = DKC * 32 + 8;
   constexpr int VS = KT + 8;
   constexpr int TP = KT / 2;                  // token pairs
   if (threadIdx.x < KT) {
     const int j = kv0 + threadIdx.x;
-    row_lds[threadIdx.x] =
-        j <= last ? (btr[j / page] * G + g) * page + (j % page) : -1;
+    const int pg = j <= last ? btr[j / page] : 0, off = j % page;
+    row_lds[threadIdx.x] = j <= last ? (pg * G + g) * page + off : -1;
+    vrow_lds[threadIdx.x] = j <= last ? (pg * GV + gv) * page + off : -1;
   }
   __syncthreads();
-  constexpr int KIT = (KT * DKC * 4 + NT - 1) / NT;
+  constexpr int KIT = (NK * KT * DKC * 4 + NT - 1) / NT;
 #pragma unroll
   for (int it = 0; it < KIT; ++it) {
     const int i = it * NT + threadIdx.x;
-    if (i >= KT * DKC * 4) break;
+    if (i >= NK * KT * DKC * 4) break;
     const int tok = i / (DKC * 4), e0 = (i % (DKC * 4)) * 8;
-    const int row = row_lds[tok];
+    const int row = row_lds[NK == 1 ? tok : tok % KT];
     s16x8 v8 = {0, 0, 0, 0, 0, 0, 0, 0};
-    if (row >= 0) v8 = load8<VEC>(kc + (size_t)row * dk, e0, dk);
+    if (row >= 0)
+      v8 = load8<VEC>(kc + (size_t)(NK == 1 ? row : row + tok / KT * page) * dk,
+                      e0, dk);
     *reinterpret_cast<s16x8*>(k_lds + tok * KS + e0) = v8;
   }
   constexpr int VIT = (TP * DVT * 2 + NT - 1) / NT;
@@ -82,7 +88,7 @@ __device__ __forceinline__ void stage_kv_tile(
     const int i = it * NT + threadIdx.x;
     if (i >= TP * DVT * 2) break;
     const int tp = i % TP, e0 = (i / TP) * 8;
-    const int ra = row_lds[tp * 2], rb = row_lds[tp * 2 + 1];
+    const int ra = vrow_lds[tp * 2], rb = vrow_lds[tp * 2 + 1];
     s16x8 a = {0, 0, 0, 0, 0, 0, 0, 0}, c8 = a;
     if (ra >= 0) a = load8<VEC>(vc + (size_t)ra * ldv, e0, dv);
     if (rb >= 0) c8 = load8<VEC>(vc + (size_t)rb * ldv, e0, dv);
@@ -99,27 +105,54 @@ __device__ __forceinline__ void stage_kv_tile(
 // staged tile serves both and one head's LDS / MFMA waits hide behind the
 // other's VALU work.  KT: keys per staged tile (64, or 32 where two heads'
 // 64-key tiles would not fit in LDS).
-template <int DKC, int DVT, bool VEC, int NH, int KT>
+//
+// DIFF: the two halves of the workgroup are the two maps of one differential
+// head: query heads and key heads are laid out [K/V head][map], both maps'
+// keys are staged over one value tile (ex.vshare == 2), and at the end the
+// second map's waves hand lam * a2 to the first map's through LDS, which
+// write (a1 - lam a2) / rms * (1 - diff) * sigmoid(gate) as head h of H.
+struct DiffTail {
+  const u16* gate;     // [T, H*dv] logits at row stride ldg, or null
+  i64 ldg;
+  float lam, diff, eps;
+};
+
+template <int DKC, int DVT, bool VEC, int NH, int KT, bool DIFF = false>
 __device__ __forceinline__ void attn_prefill_mfma_body(
     u16* __restrict__ out, const u16* __restrict__ q,
     const u16* __restrict__ kc, const u16* __restrict__ vc,
     const i32* __restrict__ bt, const i32* __restrict__ cu,
     const i32* __restrict__ q_start, const i32* __restrict__ tile_seq,
     const i32* __restrict__ tile_q0, float scale, int H, int G, int dk, int dv,
-    int page, int maxp, int chunk, int window, i64 ldq, const AttnExtra& ex) {
+    int page, int maxp, int chunk, int window, i64 ldq, const AttnExtra& ex,
+    const DiffTail& df = DiffTail{}) {
   constexpr int KS = DKC * 32 + 8;   // K row stride in LDS (elements)
   constexpr int VS = KT + 8;         // V^T / P row stride (KT tokens + pad)
   constexpr int NST = KT / 16;       // 16-key sub-tiles
   constexpr int NHF = KT / 32;       // 32-key halves of P V
-  __shared__ u16 k_lds[KT * KS];
-  __shared__ u16 v_lds[DVT * 16 * VS];
+  constexpr int NK = DIFF ? 2 : 1;
+  constexpr int XS = DVT * 16 + 4;   // row stride of the maps' exchange (floats)
+  constexpr size_t KVB = sizeof(u16) * (NK * KT * KS + DVT * 16 * VS);
+  constexpr size_t XB = DIFF ? sizeof(float) * 64 * XS : 0;
+  // K tiles, V^T tile; the maps' exchange reuses the space after the walk
+  __shared__ __align__(16) char kv_lds[KVB > XB ? KVB : XB];
+  u16* k_lds = reinterpret_cast<u16*>(kv_lds);
+  u16* v_lds = k_lds + NK * KT * KS;
   __shared__ u16 p_lds[NH * 4 * 16 * VS];
   __shared__ float bias_lds[NH * 128];  // distance bias of this tile's distances
-  __shared__ i32 row_lds[KT];        // page row of every key of the tile
+  // page rows of every key of the tile
+  __shared__ i32 row_lds[KT], vrow_lds[KT];
 
-  const int hsel = threadIdx.x >> 8;           // which of the NH heads
-  const int tile = blockIdx.x, h = blockIdx.y * NH + hsel;
-  const int g = h / (H / G);
+  const int hsel = threadIdx.x >> 8;           // which of the NH heads (maps)
+  // DIFF: H, G count heads and K/V heads, blockIdx.y is the head; h and g are
+  // this half's query head of 2H and the first of the pair's key heads of 2G
+  const int tile = blockIdx.x;
+  const int hpg = H / G;
+  const int h = DIFF ? ((int)blockIdx.y / hpg * 2 + hsel) * hpg + (int)blockIdx.y % hpg
+                     : (int)blockIdx.y * NH + hsel;
+  const int g = DIFF ? (int)blockIdx.y / hpg * 2 : h / hpg;
+  const int GK = DIFF ? 2 * G : G;
+  const int GV = GK / ex.vshare, gv = g / ex.vshare;
   const int wid = (threadIdx.x >> 6) & 3, lane = threadIdx.x & 63;
   const int b = tile_seq[tile];
   const int r0 = cu[b];
@@ -169,9 +202,9 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
   for (int kv0 = nfirst > 0 ? 0 : lo; kv0 <= p_last;
        kv0 = (kv0 < a_end && kv0 + KT >= a_end) ? b0 : kv0 + KT) {
     __syncthreads();   // fragment reads of the previous tile are done
-    stage_kv_tile<DKC, DVT, VEC, 256 * NH, KT>(k_lds, v_lds, row_lds, kc, vc,
-                                               btr, kv0, p_last, G, g, page,
-                                               dk, dv, ex.ldv);
+    stage_kv_tile<DKC, DVT, VEC, 256 * NH, KT, NK>(
+        k_lds, v_lds, row_lds, vrow_lds, kc, vc, btr, kv0, p_last, GK, g, GV,
+        gv, page, dk, dv, ex.ldv);
     // distance bias for every distance between a row and a key of the tile:
     // entry i is distance i + (p0 - kv0 - (KT-1)); keys ahead of a row are masked
     if (ex.r1 && (threadIdx.x & 255) < 63 + KT) {     // each head its own table
@@ -189,7 +222,8 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
 #pragma unroll
     for (int st = 0; st < NST; ++st) {
       s_acc[st] = f32x4{0.f, 0.f, 0.f, 0.f};
-      const u16* krow = k_lds + (st * 16 + (lane & 15)) * KS + (lane >> 4) * 8;
+      const u16* krow = k_lds + (st * 16 + (lane & 15) + (DIFF ? hsel * KT : 0)) * KS +
+                        (lane >> 4) * 8;
 #pragma unroll
       for (int c = 0; c < DKC; ++c) {
         const s16x8 kf = *reinterpret_cast<const s16x8*>(krow + c * 32);
@@ -255,6 +289,48 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
     }
   }
 
+  if constexpr (DIFF) {
+    float* xch = reinterpret_cast<float*>(kv_lds) + (wrow0 + (lane >> 4) * 4) * XS;
+    __syncthreads();                 // the last tile's fragments are read
+    if (hsel == 1 && wave_live) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float f = l[r] > 0.f ? df.lam / l[r] : 0.f;
+#pragma unroll
+        for (int dt = 0; dt < DVT; ++dt)
+          xch[r * XS + dt * 16 + (lane & 15)] = o_acc[dt][r] * f;
+      }
+    }
+    __syncthreads();
+    if (hsel == 1 || !wave_live) return;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = q0 + wrow0 + (lane >> 4) * 4 + r;
+      const float inv = l[r] > 0.f ? 1.0f / l[r] : 0.f;
+      float ss = 0.f;
+#pragma unroll
+      for (int dt = 0; dt < DVT; ++dt) {     // columns past dv are zero
+        const float a = o_acc[dt][r] * inv - xch[r * XS + dt * 16 + (lane & 15)];
+        o_acc[dt][r] = a;
+        ss += a * a;
+      }
+      const float f = (1.0f - df.diff) / sqrtf(group16_sum_f32(ss) / (float)dv + df.eps);
+      if (row >= len) continue;
+      const size_t col = (size_t)blockIdx.y * dv;
+      u16* op = out + (size_t)(r0 + row) * H * dv + col;
+      const u16* gp = df.gate + (size_t)(r0 + row) * df.ldg + col;
+#pragma unroll
+      for (int dt = 0; dt < DVT; ++dt) {
+        const int d = dt * 16 + (lane & 15);
+        if (d < dv) {
+          float v = o_acc[dt][r] * f;
+          if (df.gate) v *= __frcp_rn(1.0f + __expf(-bf2f(gp[d])));
+          op[d] = f2bf(v);
+        }
+      }
+    }
+    return;
+  }
   if (!wave_live) return;
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
@@ -294,6 +370,12 @@ attn_prefill_mfma_wide_pair_kernel(AF_APM_PARAMS) {
   attn_prefill_mfma_body<18, 32, true, 2, 32>(AF_APM_ARGS);
 }
 
+template <int DKC, int DVT, bool VEC, int KT = 64>
+__global__ void __launch_bounds__(512) diff_prefill_mfma_kernel(AF_APM_PARAMS,
+                                                                DiffTail df) {
+  attn_prefill_mfma_body<DKC, DVT, VEC, 2, KT, true>(AF_APM_ARGS, df);
+}
+
 // ------------------------------------------------ single rows, many heads
 // One token's query heads of a K/V group as the rows of the MFMA tiles: the
 // case of decode steps when many heads share one K/V head (16 heads on one
@@ -306,7 +388,7 @@ attn_prefill_mfma_wide_pair_kernel(AF_APM_PARAMS) {
 // (cheap) softmax of the 16 rows, and wave w accumulates a quarter of the
 // value columns of P V against V^T staged in LDS.  No K tile in LDS: three
 // workgroups fit a CU at value sizes up to 256.  Key splits cover multiples
-// of 64 keys; with nsplit > 1 unnormalised outputs and (max, sum) go to
+// of 64 keys; with part_o unnormalised outputs and (max, sum) go to
 // part_o [T, H, nsplit, dv] / part_ml [T, H, nsplit, 2] for the split merge.
 template <int DKC, int DVT, bool VEC>
 __global__ void __launch_bounds__(256) attn_heads_mfma_kernel(
@@ -322,11 +404,12 @@ __global__ void __launch_bounds__(256) attn_heads_mfma_kernel(
   __shared__ u16 v_lds[DVT * 16 * VS];
   __shared__ u16 p_lds[4 * 16 * VS];
   __shared__ float s_lds[16 * SS];
-  __shared__ i32 row_lds[64];
+  __shared__ i32 row_lds[64], vrow_lds[64];
 
   const int t = blockIdx.x, sp = blockIdx.z;
   const int hpg = H / G, nhb = (hpg + 15) / 16;
   const int g = blockIdx.y / nhb, hb = blockIdx.y % nhb;
+  const int GV = G / ex.vshare, gv = g / ex.vshare;
   const int hbase = g * hpg + hb * 16;
   const int nrows = min(16, hpg - hb * 16);
   const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -386,8 +469,9 @@ __global__ void __launch_bounds__(256) attn_heads_mfma_kernel(
     if (threadIdx.x < 64) {
       const int jv = kv0 + threadIdx.x;
       const int j = jv < wlo ? jv - vsh : jv;
-      row_lds[threadIdx.x] =
-          jv <= hi ? (btr[j / page] * G + g) * page + (j % page) : -1;
+      const int pg = jv <= hi ? btr[j / page] : 0, off = j % page;
+      row_lds[threadIdx.x] = jv <= hi ? (pg * G + g) * page + off : -1;
+      vrow_lds[threadIdx.x] = jv <= hi ? (pg * GV + gv) * page + off : -1;
     }
     __syncthreads();
     // ---- this wave's 16 keys: K fragments from the pages ----
@@ -408,7 +492,7 @@ __global__ void __launch_bounds__(256) attn_heads_mfma_kernel(
       const int i = it * 256 + threadIdx.x;
       if (i >= 32 * DVT * 2) break;
       const int tp = i % 32, e0 = (i / 32) * 8;
-      const int ra = row_lds[tp * 2], rb = row_lds[tp * 2 + 1];
+      const int ra = vrow_lds[tp * 2], rb = vrow_lds[tp * 2 + 1];
       s16x8 a = {0, 0, 0, 0, 0, 0, 0, 0}, c8 = a;
       if (ra >= 0) a = load8<VEC>(vc + (size_t)ra * ex.ldv, e0, dv);
       if (rb >= 0) c8 = load8<VEC>(vc + (size_t)rb * ex.ldv, e0, dv);
@@ -492,7 +576,7 @@ __global__ void __launch_bounds__(256) attn_heads_mfma_kernel(
     const int hr = (lane >> 4) * 4 + r;
     if (hr >= nrows) continue;
     const size_t th = (size_t)t * H + hbase + hr;
-    if (nsplit == 1) {
+    if (!part_o) {
       const float inv = l[r] > 0.f ? 1.0f / l[r] : 0.f;
 #pragma unroll
       for (int dw = 0; dw < DVW; ++dw) {
@@ -524,9 +608,9 @@ AF_EXPORT int afm_attn_prefill_mfma(
     const void* tile_q0, float scale, int ntiles, int H, int G, int dk, int dv,
     int page, int maxp, int chunk, int window, i64 ldq, const void* sink,
     float cap, const void* r1, const void* r2, i64 ldv, int keep_first,
-    void* stream) {
+    int vshare, void* stream) {
   if (ntiles == 0) return 0;
-  if (keep_first < 0) return 9003;
+  if (keep_first < 0 || vshare < 1 || G % vshare) return 9003;
   if (G <= 0 || H % G || dk < 1 || dv < 1) return 9003;
   if (ldv < dv || cap < 0.f || ((r1 == nullptr) != (r2 == nullptr))) return 9003;
   const bool vec = (dk % 8 == 0) && (dv % 8 == 0) && (ldq % 8 == 0) &&
@@ -537,7 +621,7 @@ AF_EXPORT int afm_attn_prefill_mfma(
   // to the row kernel
   if (dk > 576 || dv > 512 || ((dk > 128 || dv > 128) && !vec)) return 9004;
   const AttnExtra ex{(const float*)sink, (const float*)r1, (const float*)r2,
-                     cap, ldv, keep_first};
+                     cap, ldv, keep_first, vshare};
   // two heads per workgroup when a K/V group has an even number of them
   const bool pair = vec && (H / G) % 2 == 0;
   hipStream_t s = (hipStream_t)stream;
@@ -572,6 +656,38 @@ AF_EXPORT int afm_attn_prefill_mfma(
   return af_last_err();
 }
 
+// Differential attention of prompt portions: H heads of two maps on G K/V
+// heads.  q [T, 2H*dk] laid out [K/V head][map][head of the group]; key pages
+// [P, 2G, page, dk] ([K/V head][map]), value pages [P, G, page, dv]; gate
+// [T, H*dv] logits at row stride ldg (or null); out [T, H*dv].
+AF_EXPORT int afm_diff_prefill_mfma(
+    void* out, const void* q, const void* kc, const void* vc, const void* bt,
+    const void* cu, const void* q_start, const void* tile_seq,
+    const void* tile_q0, float scale, int ntiles, int H, int G, int dk, int dv,
+    int page, int maxp, int window, i64 ldq, const void* gate, i64 ldg,
+    float lam, float diff, float eps, void* stream) {
+  if (ntiles == 0) return 0;
+  if (G <= 0 || H % G || dk < 1 || dv < 1) return 9003;
+  const bool vec = (dk % 8 == 0) && (dv % 8 == 0) && (ldq % 8 == 0) &&
+                   ((uintptr_t)q % 16 == 0) && ((uintptr_t)kc % 16 == 0) &&
+                   ((uintptr_t)vc % 16 == 0);
+  // 9004 sends the caller to the row kernel
+  if (dk > 128 || dv > 256 || ((dk > 64 || dv > 128) && !vec)) return 9004;
+  const AttnExtra ex{nullptr, nullptr, nullptr, 0.f, dv, 0, 2};
+  const DiffTail df{(const u16*)gate, ldg, lam, diff, eps};
+  hipStream_t s = (hipStream_t)stream;
+#define DPM(DKC, DVT, VEC)                                                     \
+  diff_prefill_mfma_kernel<DKC, DVT, VEC><<<dim3(ntiles, H), 512, 0, s>>>(     \
+      (u16*)out, (const u16*)q, (const u16*)kc, (const u16*)vc,                \
+      (const i32*)bt, (const i32*)cu, (const i32*)q_start,                     \
+      (const i32*)tile_seq, (const i32*)tile_q0, scale, H, G, dk, dv, page,    \
+      maxp, 0, window, ldq, ex, df)
+  if (dk <= 64 && dv <= 128) { if (vec) DPM(2, 8, true); else DPM(2, 8, false); }
+  else DPM(4, 16, true);
+#undef DPM
+  return af_last_err();
+}
+
 // One row per token (decode steps): q [T, H*dk] at stride ldq, position and
 // sequence of every row in positions / row_seq.  The caller merges the key
 // splits (afm_attn_split_combine) when nsplit > 1.
@@ -580,9 +696,10 @@ AF_EXPORT int afm_attn_heads_mfma(
     const void* row_seq, const void* positions, float scale, int T, int H,
     int G, int dk, int dv, int page, int maxp, int chunk, int window, i64 ldq,
     int nsplit, void* part_o, void* part_ml, const void* sink, float cap,
-    const void* r1, const void* r2, i64 ldv, int keep_first, void* stream) {
+    const void* r1, const void* r2, i64 ldv, int keep_first, int vshare,
+    void* stream) {
   if (T == 0) return 0;
-  if (keep_first < 0) return 9003;
+  if (keep_first < 0 || vshare < 1 || G % vshare) return 9003;
   if (G <= 0 || H % G || dk < 1 || dv < 1) return 9003;
   if (ldv < dv || cap < 0.f || ((r1 == nullptr) != (r2 == nullptr))) return 9003;
   if (nsplit < 1 || nsplit > 64 || (nsplit > 1 && (!part_o || !part_ml))) return 9003;
@@ -592,7 +709,7 @@ AF_EXPORT int afm_attn_heads_mfma(
                    ((uintptr_t)vc % 16 == 0);
   if (dk > 576 || dv > 512 || ((dk > 128 || dv > 128) && !vec)) return 9004;
   const AttnExtra ex{(const float*)sink, (const float*)r1, (const float*)r2,
-                     cap, ldv, keep_first};
+                     cap, ldv, keep_first, vshare};
   const int hpg = H / G;
   dim3 grid(T, G * ((hpg + 15) / 16), nsplit), blk(256);
   hipStream_t s = (hipStream_t)stream;

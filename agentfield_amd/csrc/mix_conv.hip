@@ -34,8 +34,9 @@ inline int grid_for(i64 n) {
 // tap-major [taps, C] so that neighbouring channels load together.  Inputs
 // before the chunk come from the sequence's slot of `state`
 // [slots, taps-1, C] (the taps-1 inputs before the chunk, oldest first),
-// inputs before position 0 are zero.  One workgroup per (row, 256*V
-// channels), V channels per thread.
+// inputs before position 0 are zero.  in_bias [C] (optional) is added to
+// every input from position 0 on; the slot keeps the inputs without it.  One
+// workgroup per (row, 256*V channels), V channels per thread.
 // V consecutive channels per thread (V = 4: 8- or 16-byte accesses).
 template <typename S, int V>
 __device__ __forceinline__ void ldc(const S* p, float (&o)[4]) {
@@ -69,9 +70,10 @@ template <typename S, int V>
 __global__ void __launch_bounds__(256) causal_conv_kernel(
     S* __restrict__ out, const S* __restrict__ in, i64 ldi,
     const S* __restrict__ w, const S* __restrict__ bias,
-    const S* __restrict__ state, const i32* __restrict__ row_seq,
-    const i32* __restrict__ cu, const i32* __restrict__ q_start,
-    const i32* __restrict__ sslot, int C, int taps, int silu) {
+    const S* __restrict__ in_bias, const S* __restrict__ state,
+    const i32* __restrict__ row_seq, const i32* __restrict__ cu,
+    const i32* __restrict__ q_start, const i32* __restrict__ sslot, int C,
+    int taps, int silu) {
   const int t = blockIdx.x;
   const int c = (blockIdx.y * 256 + threadIdx.x) * V;
   if (c >= C) return;
@@ -81,6 +83,8 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(
   const S* st = state + (size_t)sslot[b] * (taps - 1) * C;
   float acc[4] = {0.f, 0.f, 0.f, 0.f};
   if (bias) ldc<S, V>(bias + c, acc);
+  float ib[4] = {0.f, 0.f, 0.f, 0.f};
+  if (in_bias) ldc<S, V>(in_bias + c, ib);
   for (int l = 0; l < taps; ++l) {        // lag
     if (pos - l < 0) break;
     float v[4], wv[4];
@@ -88,7 +92,7 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(
     else ldc<S, V>(st + (size_t)(taps - 1 - (l - k)) * C + c, v);
     ldc<S, V>(w + (size_t)(taps - 1 - l) * C + c, wv);
 #pragma unroll
-    for (int j = 0; j < V; ++j) acc[j] += wv[j] * v[j];
+    for (int j = 0; j < V; ++j) acc[j] += wv[j] * (v[j] + ib[j]);
   }
   if (silu) {
 #pragma unroll
@@ -128,7 +132,8 @@ __global__ void __launch_bounds__(256) conv_state_kernel(
 }  // namespace
 
 AF_EXPORT int afm_causal_conv(void* out, const void* in, i64 ldi,
-                              const void* w, const void* bias, void* state,
+                              const void* w, const void* bias,
+                              const void* in_bias, void* state,
                               const void* row_seq, const void* cu,
                               const void* q_start, const void* sslot, int T,
                               int B, int C, int taps, int silu, int dt,
@@ -138,13 +143,14 @@ AF_EXPORT int afm_causal_conv(void* out, const void* in, i64 ldi,
   hipStream_t s = (hipStream_t)stream;
   const bool vec = C % 4 == 0 && ldi % 4 == 0 && (uintptr_t)out % 16 == 0 &&
                    (uintptr_t)in % 16 == 0 && (uintptr_t)bias % 16 == 0 &&
-                   (uintptr_t)w % 16 == 0 &&
+                   (uintptr_t)w % 16 == 0 && (uintptr_t)in_bias % 16 == 0 &&
                    (uintptr_t)state % 16 == 0;
   const int vw = vec ? 4 : 1;
   dim3 grid(T, (C / vw + 255) / 256);
 #define CONVK(ST, V)                                                         \
   causal_conv_kernel<ST, V><<<grid, 256, 0, s>>>((ST*)out,                   \
-      (const ST*)in, ldi, (const ST*)w, (const ST*)bias, (const ST*)state,   \
+      (const ST*)in, ldi, (const ST*)w, (const ST*)bias,                     \
+      (const ST*)in_bias, (const ST*)state,                                  \
       (const i32*)row_seq, (const i32*)cu, (const i32*)q_start,              \
       (const i32*)sslot, C, taps, silu)
 #define CONV(ST)                                                             \

@@ -180,17 +180,207 @@ __global__ void __launch_bounds__(256) scatter_state_kernel(
 template <typename S>
 __global__ void __launch_bounds__(256) norm_rows_kernel(
     S* __restrict__ out, const float* __restrict__ x, const S* __restrict__ w,
-    const i32* __restrict__ rows, float eps, int W, int one_plus) {
+    const i32* __restrict__ rows, float eps, int W, int one_plus, int center) {
   __shared__ float red[4];
   const int r = blockIdx.x;
   const float* xr = x + (size_t)(rows ? rows[r] : r) * W;
+  float mean = 0.f;
+  if (center) {
+    float sm[1] = {0.f};
+    for (int i = threadIdx.x; i < W; i += 256) sm[0] += xr[i];
+    block_sum<1>(sm, red);
+    mean = sm[0] / (float)W;
+  }
   float ss[1] = {0.f};
-  for (int i = threadIdx.x; i < W; i += 256) ss[0] += xr[i] * xr[i];
+  for (int i = threadIdx.x; i < W; i += 256) ss[0] += (xr[i] - mean) * (xr[i] - mean);
   block_sum<1>(ss, red);
   const float rs = 1.0f / sqrtf(ss[0] / (float)W + eps);
   for (int i = threadIdx.x; i < W; i += 256) {
     const float g = ldf<S>(w + i) + (one_plus ? 1.0f : 0.f);
-    stf<S>(out + (size_t)r * W + i, xr[i] * rs * g);
+    stf<S>(out + (size_t)r * W + i, (xr[i] - mean) * rs * g);
+  }
+}
+
+// Layer norms on both sides of a sublayer, in one pass over the row:
+//   x += mult * LN(y) * w_post        (y given: the previous sublayer's output)
+//   h  = LN(x) * w_pre                (h given: the next sublayer's input)
+// LN(u) = (u - mean) / sqrt(mean((u - mean)^2) + eps), the variance taken
+// from the deviations in a second sum.  x is the fp32 residual, y in Y.
+// REG: the row fits 4 passes of the workgroup and waits in registers between
+// the sums; otherwise it is read again (x through memory).
+constexpr int SWN_IT = 4;
+
+template <typename S, typename Y, int V, int NT, bool REG>
+__global__ void __launch_bounds__(NT) sandwich_norm_kernel(
+    float* __restrict__ x, S* __restrict__ h, const Y* __restrict__ y,
+    i64 ldy, const S* __restrict__ w_post, const S* __restrict__ w_pre,
+    float mult, float eps, int W) {
+  __shared__ float red[NT / 64];
+  const int t = blockIdx.x;
+  float* xr = x + (size_t)t * W;
+  auto total = [&](float v) {                // fixed order, every thread
+    v = wave_sum_f32(v);
+    __syncthreads();                         // red may still be read
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < NT / 64; ++i) s += red[i];
+    return s;
+  };
+  const float inv_w = 1.0f / (float)W;
+  if constexpr (REG) {
+    float xv[SWN_IT][4], uv[SWN_IT][4];
+    float s = 0.f;
+#pragma unroll
+    for (int p = 0; p < SWN_IT; ++p) {
+      const int i = (p * NT + threadIdx.x) * V;
+      if (i < W) {
+        ldv<float, V>(xr + i, xv[p]);
+        if (y) {
+          ldv<Y, V>(y + (size_t)t * ldy + i, uv[p]);
+#pragma unroll
+          for (int j = 0; j < V; ++j) s += uv[p][j];
+        }
+      }
+    }
+    if (y) {
+      const float mean = total(s) * inv_w;
+      s = 0.f;
+#pragma unroll
+      for (int p = 0; p < SWN_IT; ++p) {
+        const int i = (p * NT + threadIdx.x) * V;
+        if (i < W) {
+#pragma unroll
+          for (int j = 0; j < V; ++j) {
+            uv[p][j] -= mean;
+            s += uv[p][j] * uv[p][j];
+          }
+        }
+      }
+      const float f = mult / sqrtf(total(s) * inv_w + eps);
+#pragma unroll
+      for (int p = 0; p < SWN_IT; ++p) {
+        const int i = (p * NT + threadIdx.x) * V;
+        if (i < W) {
+          float wv[4];
+          ldv<S, V>(w_post + i, wv);
+#pragma unroll
+          for (int j = 0; j < V; ++j) xv[p][j] += uv[p][j] * f * wv[j];
+          stv<float, V>(xr + i, xv[p]);
+        }
+      }
+    }
+    if (!h) return;
+    s = 0.f;
+#pragma unroll
+    for (int p = 0; p < SWN_IT; ++p) {
+      const int i = (p * NT + threadIdx.x) * V;
+      if (i < W) {
+#pragma unroll
+        for (int j = 0; j < V; ++j) s += xv[p][j];
+      }
+    }
+    const float mean = total(s) * inv_w;
+    s = 0.f;
+#pragma unroll
+    for (int p = 0; p < SWN_IT; ++p) {
+      const int i = (p * NT + threadIdx.x) * V;
+      if (i < W) {
+#pragma unroll
+        for (int j = 0; j < V; ++j) {
+          xv[p][j] -= mean;
+          s += xv[p][j] * xv[p][j];
+        }
+      }
+    }
+    const float rs = 1.0f / sqrtf(total(s) * inv_w + eps);
+#pragma unroll
+    for (int p = 0; p < SWN_IT; ++p) {
+      const int i = (p * NT + threadIdx.x) * V;
+      if (i < W) {
+        float wv[4];
+        ldv<S, V>(w_pre + i, wv);
+#pragma unroll
+        for (int j = 0; j < V; ++j) wv[j] *= xv[p][j] * rs;
+        stv<S, V>(h + (size_t)t * W + i, wv);
+      }
+    }
+  } else {
+    float v[4], wv[4], u[4];
+    float s = 0.f;
+    if (y) {
+      const Y* yr = y + (size_t)t * ldy;
+      for (int i = threadIdx.x * V; i < W; i += NT * V) {
+        ldv<Y, V>(yr + i, u);
+#pragma unroll
+        for (int j = 0; j < V; ++j) s += u[j];
+      }
+      const float mean = total(s) * inv_w;
+      s = 0.f;
+      for (int i = threadIdx.x * V; i < W; i += NT * V) {
+        ldv<Y, V>(yr + i, u);
+#pragma unroll
+        for (int j = 0; j < V; ++j) s += (u[j] - mean) * (u[j] - mean);
+      }
+      const float f = mult / sqrtf(total(s) * inv_w + eps);
+      for (int i = threadIdx.x * V; i < W; i += NT * V) {
+        ldv<Y, V>(yr + i, u);
+        ldv<S, V>(w_post + i, wv);
+        ldv<float, V>(xr + i, v);
+#pragma unroll
+        for (int j = 0; j < V; ++j) v[j] += (u[j] - mean) * f * wv[j];
+        stv<float, V>(xr + i, v);            // read back by the same thread
+      }
+    }
+    if (!h) return;
+    s = 0.f;
+    for (int i = threadIdx.x * V; i < W; i += NT * V) {
+      ldv<float, V>(xr + i, v);
+#pragma unroll
+      for (int j = 0; j < V; ++j) s += v[j];
+    }
+    const float mean = total(s) * inv_w;
+    s = 0.f;
+    for (int i = threadIdx.x * V; i < W; i += NT * V) {
+      ldv<float, V>(xr + i, v);
+#pragma unroll
+      for (int j = 0; j < V; ++j) s += (v[j] - mean) * (v[j] - mean);
+    }
+    const float rs = 1.0f / sqrtf(total(s) * inv_w + eps);
+    for (int i = threadIdx.x * V; i < W; i += NT * V) {
+      ldv<float, V>(xr + i, v);
+      ldv<S, V>(w_pre + i, wv);
+#pragma unroll
+      for (int j = 0; j < V; ++j) wv[j] *= (v[j] - mean) * rs;
+      stv<S, V>(h + (size_t)t * W + i, wv);
+    }
+  }
+}
+
+// xIELU: z > 0: cp z^2 + z/2;  z <= 0: cn (e^z - 1 - z) + z/2, with (cp, cn)
+// in coef.  bf16 storage takes the hardware exponential.
+template <typename S, int V>
+__global__ void __launch_bounds__(256) xielu_kernel(
+    S* __restrict__ out, const S* __restrict__ z, i64 ldz,
+    const float* __restrict__ coef, int T, int F) {
+  const float cp = coef[0], cn = coef[1];
+  const i64 per = F / V;
+  const i64 total = (i64)T * per;
+  for (i64 i = (i64)blockIdx.x * 256 + threadIdx.x; i < total;
+       i += (i64)gridDim.x * 256) {
+    const i64 t = i / per;
+    const int c = (int)(i % per) * V;
+    float v[4];
+    ldv<S, V>(z + t * ldz + c, v);
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      const float a = v[j];
+      const float n = fminf(a, 0.f);
+      const float e = sizeof(S) == 2 ? __expf(n) - 1.0f : expm1f(n);
+      v[j] = (a > 0.f ? cp * a * a : cn * (e - n)) + 0.5f * a;
+    }
+    stv<S, V>(out + t * F + c, v);
   }
 }
 
@@ -577,14 +767,14 @@ AF_EXPORT int afm_scatter_state(void* prev, const void* last,
 
 AF_EXPORT int afm_norm_rows(void* out, const void* x, const void* w,
                             const void* rows, float eps, int R, int W,
-                            int one_plus, int dt, void* stream) {
+                            int one_plus, int center, int dt, void* stream) {
   if (R == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   MIX_DISPATCH(dt,
       (norm_rows_kernel<u16><<<R, 256, 0, s>>>((u16*)out, (const float*)x,
-          (const u16*)w, (const i32*)rows, eps, W, one_plus)),
+          (const u16*)w, (const i32*)rows, eps, W, one_plus, center)),
       (norm_rows_kernel<float><<<R, 256, 0, s>>>((float*)out, (const float*)x,
-          (const float*)w, (const i32*)rows, eps, W, one_plus)));
+          (const float*)w, (const i32*)rows, eps, W, one_plus, center)));
   return af_last_err();
 }
 
@@ -691,6 +881,56 @@ AF_EXPORT int afm_norm_residual(void* x, void* h, const void* y, i64 ldy,
   else if (dt == 1) NR(float, float);
   else return 9002;
 #undef NR
+  return af_last_err();
+}
+
+// x [T, W] fp32 in place; y (or null) at row stride ldy, fp32 when y_f32; h
+// (or null) [T, W] in the storage dtype.
+AF_EXPORT int afm_sandwich_norm(void* x, void* h, const void* y, i64 ldy,
+                                int y_f32, const void* w_post,
+                                const void* w_pre, float mult, float eps,
+                                int T, int W, int dt, void* stream) {
+  if (T == 0) return 0;
+  if ((y && !w_post) || (h && !w_pre)) return 9003;
+  hipStream_t s = (hipStream_t)stream;
+  const bool vec = W % 4 == 0 && ldy % 4 == 0 && aligned16(x, h, y, w_post, w_pre);
+  const int cols = W / (vec ? 4 : 1);
+  // few rows of many columns: one column group per thread
+  const bool wide = T <= 512 && cols > 256;
+#define SWK(ST, YT, V, NT, R)                                                \
+  sandwich_norm_kernel<ST, YT, V, NT, R><<<T, NT, 0, s>>>((float*)x, (ST*)h, \
+      (const YT*)y, ldy, (const ST*)w_post, (const ST*)w_pre, mult, eps, W)
+#define SWR(ST, YT, V)                                                       \
+  do {                                                                       \
+    if (wide && cols <= SWN_IT * 1024) SWK(ST, YT, V, 1024, true);           \
+    else if (!wide && cols <= SWN_IT * 256) SWK(ST, YT, V, 256, true);       \
+    else SWK(ST, YT, V, 256, false);                                         \
+  } while (0)
+#define SW(ST, YT)                                                           \
+  do { if (vec) SWR(ST, YT, 4); else SWR(ST, YT, 1); } while (0)
+  if (dt == 0) { if (y_f32) SW(u16, float); else SW(u16, u16); }
+  else if (dt == 1) SW(float, float);
+  else return 9002;
+#undef SW
+#undef SWR
+#undef SWK
+  return af_last_err();
+}
+
+AF_EXPORT int afm_xielu(void* out, const void* z, i64 ldz, const void* coef,
+                        int T, int F, int dt, void* stream) {
+  if (T == 0 || F == 0) return 0;
+  hipStream_t s = (hipStream_t)stream;
+  const bool vec = F % 4 == 0 && ldz % 4 == 0 && aligned16(out, z);
+  const i64 total = (i64)T * (vec ? F / 4 : F);
+  const int grid = (int)((total + 255) / 256 < 16384 ? (total + 255) / 256 : 16384);
+#define XI(S, V)                                                             \
+  xielu_kernel<S, V><<<grid, 256, 0, s>>>((S*)out, (const S*)z, ldz,         \
+                                          (const float*)coef, T, F)
+  if (dt == 0) { if (vec) XI(u16, 4); else XI(u16, 1); }
+  else if (dt == 1) { if (vec) XI(float, 4); else XI(float, 1); }
+  else return 9002;
+#undef XI
   return af_last_err();
 }
 

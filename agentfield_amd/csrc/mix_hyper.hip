@@ -1,8 +1,7 @@
 // Glue of hyper-connected decoders: several fp32 residual streams per token
 // mixed by small learned matrices, an RMSNorm and a short causal convolution
-// in front of every sublayer, and the row-wise steps of latent attention
-// (latent norm, interleaved rotary positions, cache append, query assembly,
-// gated head outputs).
+// in front of every sublayer (the row steps of latent attention live in
+// mix_latent.hip).
 //
 // Storage dtype S is bf16 (raw u16) or fp32.  The streams, norm statistics,
 // convolution inputs and sums, angles and gates are fp32; S is what the
@@ -52,16 +51,7 @@ __device__ __forceinline__ void stv(S* p, const float (&o)[4]) {
   }
 }
 
-__device__ __forceinline__ float block_sum_256(float v, float* red) {
-  v = wave_sum_f32(v);
-  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
-  __syncthreads();
-  const float s = red[0] + red[1] + red[2] + red[3];
-  __syncthreads();
-  return s;
-}
-
-// the same for NT threads (a multiple of 64, at most 1024), fixed order
+// block-wide sum over NT threads (a multiple of 64, at most 1024), fixed order
 template <int NT>
 __device__ __forceinline__ float block_sum(float v, float* red) {
   v = wave_sum_f32(v);
@@ -306,93 +296,6 @@ __global__ void __launch_bounds__(256) canon_state_kernel(
   }
 }
 
-// ------------------------------------------------------- latent attention
-// One workgroup per row.  The down projection's row holds the latent (first
-// R values) and one rotary key part (rd values); the latent is RMS-normed
-// with a plain weight, the key part rotated, and [latent | key part] goes to
-// the key pages [P, 1, page, R + rd] at `slot`.  The attention query of head
-// h is [q in latent space (R, already in place) | rotate(q[t, h, dim:dim+rd])]:
-// the kernel fills the rotary slices of qf [T, H, R + rd].  Rotation pairs
-// element 2i with 2i+1 for i < rot/2, angle = position * inv_freq[i] in fp32.
-template <typename S>
-__global__ void __launch_bounds__(256) latent_prep_kernel(
-    S* __restrict__ qf, S* __restrict__ kc, const S* __restrict__ q, i64 ldq,
-    const S* __restrict__ dkv, i64 lddkv,
-    const S* __restrict__ normw, const float* __restrict__ inv_freq,
-    const i32* __restrict__ positions, const i64* __restrict__ slots,
-    float eps, int T, int H, int dim, int rd, int R, int rot) {
-  __shared__ float red[4];
-  extern __shared__ float cs[];              // [rot/2] cos, [rot/2] sin
-  const int t = blockIdx.x;
-  const int half = rot / 2;
-  const float pos = (float)positions[t];
-  for (int i = threadIdx.x; i < half; i += 256) {
-    float sn, c;
-    sincosf(pos * inv_freq[i], &sn, &c);
-    cs[i] = c;
-    cs[half + i] = sn;
-  }
-  const S* dr = dkv + (size_t)t * lddkv;
-  float ss = 0.f;
-  for (int i = threadIdx.x; i < R; i += 256) {
-    const float v = ldf<S>(dr + i);
-    ss += v * v;
-  }
-  const float rinv = 1.0f / sqrtf(block_sum_256(ss, red) / (float)R + eps);
-  const i64 sl = slots[t];
-  const int dkc = R + rd;
-  if (sl >= 0) {
-    S* kr = kc + (size_t)sl * dkc;           // one K/V head: slot * row
-    for (int i = threadIdx.x; i < R; i += 256)
-      stf<S>(kr + i, ldf<S>(dr + i) * rinv * ldf<S>(normw + i));
-    for (int i = threadIdx.x; i < rd; i += 256) {
-      float v = ldf<S>(dr + R + i);
-      if (i < rot) {
-        const int pr = i >> 1;
-        const float o = ldf<S>(dr + R + (i ^ 1));
-        v = (i & 1) ? v * cs[pr] + o * cs[half + pr]
-                    : v * cs[pr] - o * cs[half + pr];
-      }
-      stf<S>(kr + R + i, v);
-    }
-  }
-  const int dq = dim + rd;
-  for (int i = threadIdx.x; i < H * rd; i += 256) {
-    const int h = i / rd, k = i % rd;
-    const S* qr = q + (size_t)t * ldq + (size_t)h * dq + dim;
-    float v = ldf<S>(qr + k);
-    if (k < rot) {
-      const int pr = k >> 1;
-      const float o = ldf<S>(qr + (k ^ 1));
-      v = (k & 1) ? v * cs[pr] + o * cs[half + pr]
-                  : v * cs[pr] - o * cs[half + pr];
-    }
-    stf<S>(qf + ((size_t)t * H + h) * dkc + R + k, v);
-  }
-}
-
-// out[t, h*dv + d] = o[h, t, d] * sigmoid(g[t, h*dv + d]): head-major
-// per-head results back to token rows, times the output gate.
-template <typename S, int V>
-__global__ void __launch_bounds__(256) gate_heads_kernel(
-    S* __restrict__ out, const S* __restrict__ o, const S* __restrict__ g,
-    i64 ldg, int T, int H, int dv) {
-  const int per = dv / V;
-  const i64 total = (i64)T * H * per;
-  for (i64 i = (i64)blockIdx.x * 256 + threadIdx.x; i < total;
-       i += (i64)gridDim.x * 256) {
-    const int d = (int)(i % per) * V;
-    const int h = (int)((i / per) % H);
-    const i64 t = i / ((i64)per * H);
-    float gv[4], ov[4];
-    ldv<S, V>(g + t * ldg + (i64)h * dv + d, gv);
-    ldv<S, V>(o + ((i64)h * T + t) * dv + d, ov);
-#pragma unroll
-    for (int j = 0; j < V; ++j) ov[j] = ov[j] / (1.0f + expf(-gv[j]));
-    stv<S, V>(out + (t * H + h) * dv + d, ov);
-  }
-}
-
 // out = max(z, 0)^2, rows of z at stride ldz.
 template <typename S, int V>
 __global__ void __launch_bounds__(256) relu2_kernel(
@@ -519,49 +422,6 @@ AF_EXPORT int afm_canon_conv(void* h, const void* n, const void* w,
     canon_state_kernel<<<dim3(B, (W + 255) / 256), 256, 0, s>>>(
         (float*)state, (const float*)n, (const i32*)cu, (const i32*)q_start,
         (const i32*)sslot, W, taps);
-  return af_last_err();
-}
-
-AF_EXPORT int afm_latent_prep(void* qf, void* kc, const void* q, i64 ldq,
-                              const void* dkv, i64 lddkv,
-                              const void* normw, const void* inv_freq,
-                              const void* positions, const void* slots,
-                              float eps, int T, int H, int dim, int rd, int R,
-                              int rot, int dt, void* stream) {
-  if (T == 0) return 0;
-  if (rot < 0 || rot > rd || (rot & 1) || (rot && !inv_freq)) return 9003;
-  hipStream_t s = (hipStream_t)stream;
-  const size_t sm = (size_t)(rot > 0 ? rot : 1) * sizeof(float);
-  if (dt == 0)
-    latent_prep_kernel<u16><<<T, 256, sm, s>>>(
-        (u16*)qf, (u16*)kc, (const u16*)q, ldq, (const u16*)dkv, lddkv,
-        (const u16*)normw, (const float*)inv_freq,
-        (const i32*)positions, (const i64*)slots, eps, T, H, dim, rd, R, rot);
-  else if (dt == 1)
-    latent_prep_kernel<float><<<T, 256, sm, s>>>(
-        (float*)qf, (float*)kc, (const float*)q, ldq, (const float*)dkv, lddkv,
-        (const float*)normw, (const float*)inv_freq,
-        (const i32*)positions, (const i64*)slots, eps, T, H, dim, rd, R, rot);
-  else
-    return 9002;
-  return af_last_err();
-}
-
-AF_EXPORT int afm_gate_heads(void* out, const void* o, const void* g, i64 ldg,
-                             int T, int H, int dv, int dt, void* stream) {
-  if (T == 0) return 0;
-  hipStream_t s = (hipStream_t)stream;
-  const bool vec = dv % 4 == 0 && ldg % 4 == 0 && al16(out) && al16(o) &&
-                   al16(g);
-  const i64 total = (i64)T * H * (vec ? dv / 4 : dv);
-  const int grid = (int)((total + 255) / 256 < 16384 ? (total + 255) / 256 : 16384);
-#define GH(S, V)                                                              \
-  gate_heads_kernel<S, V><<<grid, 256, 0, s>>>((S*)out, (const S*)o,          \
-                                               (const S*)g, ldg, T, H, dv)
-  if (dt == 0) { if (vec) GH(u16, 4); else GH(u16, 1); }
-  else if (dt == 1) { if (vec) GH(float, 4); else GH(float, 1); }
-  else return 9002;
-#undef GH
   return af_last_err();
 }
 

@@ -128,7 +128,8 @@ __global__ void __launch_bounds__(256) masked_attention_kernel(
     const S* __restrict__ vc, const i32* __restrict__ bt,
     const i32* __restrict__ row_seq, const i32* __restrict__ positions,
     float scale, int n_rh, int H, int G, int dk, int dv, int page, int maxp,
-    int chunk, int window, i64 ldq, AttnExtra ex) {
+    int chunk, int window, i64 ldq, float* __restrict__ part_o,
+    float* __restrict__ part_ml, AttnExtra ex) {
   extern __shared__ float smem[];           // [4][dk + 64]
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int rh = blockIdx.x * 4 + wave;
@@ -137,6 +138,7 @@ __global__ void __launch_bounds__(256) masked_attention_kernel(
   float* ps = qs + dk;
   const int t = rh / H, h = rh % H;
   const int g = h / (H / G);
+  const int GV = G / ex.vshare, gv = g / ex.vshare;
   const int pos = positions[t];
   const i32* btr = bt + (size_t)row_seq[t] * maxp;
   int lo = 0;
@@ -183,11 +185,23 @@ __global__ void __launch_bounds__(256) masked_attention_kernel(
         for (int jj = 0; jj < cnt; ++jj) {
           const int jk = (j0 + jj) < lo ? j0 + jj - vsh : j0 + jj;
           const int pg = btr[jk / page];
-          a += ps[jj] * ldf<S>(vc + (((size_t)pg * G + g) * page + (jk % page)) * ex.ldv + d);
+          a += ps[jj] * ldf<S>(vc + (((size_t)pg * GV + gv) * page + (jk % page)) * ex.ldv + d);
         }
       }
       acc[i] = a;
     }
+  }
+  if (part_o) {                              // one unnormalised part per row
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i) {
+      const int d = lane + 64 * i;
+      if (d < dv) part_o[(size_t)rh * dv + d] = acc[i];
+    }
+    if (lane == 0) {
+      part_ml[(size_t)rh * 2] = m;
+      part_ml[(size_t)rh * 2 + 1] = l;
+    }
+    return;
   }
   const float inv = 1.0f / l;
 #pragma unroll
@@ -244,9 +258,9 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(
     int window, i64 ldq, int lpk_log2, int lpv_log2, int kt, int nsplit,
     float* __restrict__ part_o, float* __restrict__ part_ml, AttnExtra ex) {
   // nsplit > 1: the visible keys are cut into nsplit ranges, one workgroup
-  // each (grid.z = head blocks x nsplit); unnormalised outputs and (max,
-  // sum) go to part_o [T, H, nsplit, dv] / part_ml [T, H, nsplit, 2] and
-  // attn_split_combine_kernel merges them.
+  // each (grid.z = head blocks x nsplit).  With part_o, unnormalised outputs
+  // and (max, sum) go to part_o [T, H, nsplit, dv] / part_ml [T, H, nsplit,
+  // 2] for attn_split_combine_kernel (or diff_combine_kernel) to merge.
   constexpr int EPL = 16 / sizeof(S);
   extern __shared__ float smem[];
   const int dvp = EPL << lpv_log2;             // padded value width
@@ -260,6 +274,7 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(
   const int dkp = (dk + EPL - 1) / EPL * EPL;
   float* qs = r2s + 8;                         // [GQ][dkp] scaled queries
   const int t = blockIdx.x, g = blockIdx.y;
+  const int GV = G / ex.vshare, gv = g / ex.vshare;
   const int hpg = H / G;
   const int zh = blockIdx.z / nsplit, sp = blockIdx.z % nsplit;
   const int h0 = g * hpg + zh * GQ;
@@ -372,7 +387,7 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(
       for (int u = 0; u < 4; ++u) {
         const int jv = tile0 + min(kb + u * 4 * kpv + kiv, nk - 1);
         const int j = jv < wlo ? jv - vsh : jv;
-        const S* vr = vc + (((size_t)btr[j / page] * G + g) * page + (j % page)) * ex.ldv;
+        const S* vr = vc + (((size_t)btr[j / page] * GV + gv) * page + (j % page)) * ex.ldv;
         load_slice<S, VEC>(vr, liv * EPL, dv, vv[u]);
       }
 #pragma unroll
@@ -404,12 +419,12 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(
     float o = 0.f;
 #pragma unroll
     for (int w = 0; w < 4; ++w) o += red[(w * GQ + gg) * dvp + d];
-    if (nsplit == 1)
+    if (!part_o)
       stf<S>(out + ((size_t)t * H + h0 + gg) * dv + d, o / l_run[gg]);
     else
       part_o[(((size_t)t * H + h0 + gg) * nsplit + sp) * dv + d] = o;
   }
-  if (nsplit > 1 && threadIdx.x < nh) {
+  if (part_o && threadIdx.x < nh) {
     float* ml = part_ml + (((size_t)t * H + h0 + threadIdx.x) * nsplit + sp) * 2;
     ml[0] = m_run[threadIdx.x];
     ml[1] = l_run[threadIdx.x];
@@ -441,6 +456,56 @@ __global__ void __launch_bounds__(256) attn_split_combine_kernel(
         o += part_o[((size_t)rh * nsplit + s) * dv + d] * ws;
     }
     if (d < dv) stf<S>(out + (size_t)rh * dv + d, o * inv);
+  }
+}
+
+// One wave per (row, head of a differential attention): merge the key splits
+// of both maps, o = a1 - lam a2, o <- o / rms(o) * (1 - diff), times
+// sigmoid(gate) per element (gate null: none).  The maps' query heads are
+// laid out [K/V head][map][head of the group].
+template <typename S, int NV>
+__global__ void __launch_bounds__(256) diff_combine_kernel(
+    S* __restrict__ out, const float* __restrict__ part_o,
+    const float* __restrict__ part_ml, const S* __restrict__ gate, i64 ldg,
+    float lam, float diff, float eps, int n_rh, int H, int hpg, int nsplit,
+    int dv) {
+  const int rh = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (rh >= n_rh) return;
+  const int lane = threadIdx.x & 63;
+  const int t = rh / H, h = rh % H;
+  const int g = h / hpg, hg = h % hpg;
+  float o[NV];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) o[i] = 0.f;
+#pragma unroll
+  for (int mp = 0; mp < 2; ++mp) {
+    const size_t ph = (size_t)t * 2 * H + (size_t)(g * 2 + mp) * hpg + hg;
+    const float* ml = part_ml + ph * nsplit * 2;
+    const float ms = lane < nsplit ? ml[2 * lane] : AF_NEG_INF;
+    const float ls = lane < nsplit ? ml[2 * lane + 1] : 0.f;
+    const float m = wave_max_f32(ms);
+    const float w = ms > AF_NEG_INF ? expf(ms - m) : 0.f;
+    const float ws = (mp ? -lam : 1.0f) * w / wave_sum_f32(w * ls);
+    for (int s = 0; s < nsplit; ++s) {
+      if (__shfl(w, s, 64) <= 0.f) continue;   // empty splits are never read
+      const float wv = __shfl(ws, s, 64);
+      const float* p = part_o + (ph * nsplit + s) * dv;
+#pragma unroll
+      for (int i = 0; i < NV; ++i)
+        if (i * 64 + lane < dv) o[i] += wv * p[i * 64 + lane];
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) ss += o[i] * o[i];
+  const float f = (1.0f - diff) / sqrtf(wave_sum_f32(ss) / (float)dv + eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int d = i * 64 + lane;
+    if (d >= dv) continue;
+    float v = o[i] * f;
+    if (gate) v /= 1.0f + expf(-ldf<S>(gate + (size_t)t * ldg + (size_t)h * dv + d));
+    stf<S>(out + (size_t)rh * dv + d, v);
   }
 }
 
@@ -694,7 +759,6 @@ static int launch_attention(void* out, const void* q, const void* kc,
                        (size_t)gq * dkp) * sizeof(float);
     const bool vec = dk % EPL == 0 && dv % EPL == 0 && ex.ldv % EPL == 0 &&
                      (uintptr_t)kc % 16 == 0 && (uintptr_t)vc % 16 == 0;
-    if (nsplit < 1 || nsplit > 64 || (nsplit > 1 && (!part_o || !part_ml))) return 9003;
     dim3 grid(T, G, ((hpg + gq - 1) / gq) * nsplit);
 #define ROWS(GQ, VEC)                                                         \
   attn_rows_kernel<S, GQ, VEC><<<grid, 256, sm, s>>>(                         \
@@ -709,12 +773,13 @@ static int launch_attention(void* out, const void* q, const void* kc,
       else if (gq == 4) ROWS(4, false); else ROWS(8, false);
     }
 #undef ROWS
-    if (nsplit > 1)
+    if (nsplit > 1 && out)
       attn_split_combine_kernel<S><<<(T * H + 3) / 4, 256, 0, s>>>(
           (S*)out, part_o, part_ml, T * H, nsplit, dv);
     return af_last_err();
   }
-  // very wide heads: one wave per (row, head), scalar key walk
+  // very wide heads: one wave per (row, head), scalar key walk, no key splits
+  if (!out && nsplit > 1) return 9003;
   const int n_rh = T * H;
   const int grid = (n_rh + 3) / 4;
   const size_t sm = (size_t)4 * (dk + 64) * sizeof(float);
@@ -722,7 +787,8 @@ static int launch_attention(void* out, const void* q, const void* kc,
   masked_attention_kernel<S, MV><<<grid, 256, sm, s>>>(                      \
       (S*)out, (const S*)q, (const S*)kc, (const S*)vc, (const i32*)bt,      \
       (const i32*)row_seq, (const i32*)positions, scale, n_rh, H, G, dk, dv, \
-      page, maxp, chunk, window, ldq, ex)
+      page, maxp, chunk, window, ldq, out ? nullptr : part_o,                \
+      out ? nullptr : part_ml, ex)
   if (dv <= 64) ATT(1);
   else if (dv <= 128) ATT(2);
   else if (dv <= 256) ATT(4);
@@ -732,19 +798,23 @@ static int launch_attention(void* out, const void* q, const void* kc,
   return af_last_err();
 }
 
+// out null: the unmerged partial softmaxes stay in part_o / part_ml.
 AF_EXPORT int afm_masked_attention(
     void* out, const void* q, const void* kc, const void* vc, const void* bt,
     const void* row_seq, const void* positions, float scale, int T, int H,
     int G, int dk, int dv, int page, int maxp, int chunk, int window, i64 ldq,
     int nsplit, void* part_o, void* part_ml, const void* sink, float cap,
-    const void* r1, const void* r2, i64 ldv, int keep_first, int dt,
-    void* stream) {
+    const void* r1, const void* r2, i64 ldv, int keep_first, int vshare,
+    int dt, void* stream) {
   if (T == 0) return 0;
   if (G <= 0 || H % G || dv > 1024 || dk > 2048) return 9003;
+  if (vshare < 1 || G % vshare) return 9003;
+  if (nsplit < 1 || nsplit > 64 ||
+      ((nsplit > 1 || !out) && (!part_o || !part_ml))) return 9003;
   if (ldv < dv || cap < 0.f || ((r1 == nullptr) != (r2 == nullptr))) return 9003;
   if (keep_first < 0) return 9003;
   const AttnExtra ex{(const float*)sink, (const float*)r1, (const float*)r2,
-                     cap, ldv, keep_first};
+                     cap, ldv, keep_first, vshare};
   hipStream_t s = (hipStream_t)stream;
   if (dt == 0)
     return launch_attention<u16>(out, q, kc, vc, bt, row_seq, positions, scale,
@@ -757,6 +827,39 @@ AF_EXPORT int afm_masked_attention(
                                    window, ldq, nsplit, (float*)part_o,
                                    (float*)part_ml, ex, s);
   return 9002;
+}
+
+// out [T, H*dv] from the partial softmaxes of 2H query heads laid out [key
+// head pair][map][head of the group] (part_o [T, 2H, nsplit, dv], part_ml
+// [T, 2H, nsplit, 2]); hpg query heads per K/V head.
+AF_EXPORT int afm_diff_combine(void* out, const void* part_o,
+                               const void* part_ml, const void* gate, i64 ldg,
+                               float lam, float diff, float eps, int T, int H,
+                               int hpg, int nsplit, int dv, int dt,
+                               void* stream) {
+  if (T == 0) return 0;
+  if (nsplit < 1 || nsplit > 64 || hpg < 1 || H % hpg) return 9003;
+  hipStream_t s = (hipStream_t)stream;
+  const int n_rh = T * H;
+#define DC(ST, NV)                                                            \
+  diff_combine_kernel<ST, NV><<<(n_rh + 3) / 4, 256, 0, s>>>((ST*)out,        \
+      (const float*)part_o, (const float*)part_ml, (const ST*)gate, ldg, lam, \
+      diff, eps, n_rh, H, hpg, nsplit, dv)
+#define DCV(ST)                                                               \
+  do {                                                                        \
+    if (dv <= 64) DC(ST, 1);                                                  \
+    else if (dv <= 128) DC(ST, 2);                                            \
+    else if (dv <= 256) DC(ST, 4);                                            \
+    else if (dv <= 512) DC(ST, 8);                                            \
+    else DC(ST, 16);                                                          \
+  } while (0)
+  if (dv > 1024) return 9003;
+  if (dt == 0) DCV(u16);
+  else if (dt == 1) DCV(float);
+  else return 9002;
+#undef DCV
+#undef DC
+  return af_last_err();
 }
 
 // out [T*H, dv] bf16 from part_o [T*H, nsplit, dv] / part_ml [T*H, nsplit, 2].

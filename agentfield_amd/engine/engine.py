@@ -441,6 +441,9 @@ class LLMEngine:
             self.sched.reserve(seq, len(toks))
         ids_t, pos_t, md, cu_list = self._chunk_batch(
             seqs, [s.num_tokens for s in seqs], [e[1] for e in entries])
+        if self.stateful and all(len(e[1]) == 1 for e in entries):
+            # one token per request: the batch a decode step runs
+            md.is_prefill, md.seq_lens = False, None
         rows = [cu_list[i] + w for i, e in enumerate(entries) for w in e[2]]
         self.metrics["steps"] += 1
         self.metrics["prefill_tokens"] += cu_list[-1]

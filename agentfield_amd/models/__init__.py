@@ -3,6 +3,7 @@ from .hybrid import HYBRID_CONFIGS, ReperaxConfig, ReperaxForCausalLM
 from .zudisun import ZUDISUN_CONFIGS, ZudisunConfig, ZudisunForCausalLM
 from .fugevik import FUGEVIK_CONFIGS, FugevikConfig, FugevikForCausalLM
 from .vabedra import VABEDRA_CONFIGS, VabedraConfig, VabedraForCausalLM
+from .fironex import FIRONEX_CONFIGS, FironexConfig, FironexForCausalLM
 from .registry import (architecture_of, build_model, load_model,
                        register_architecture)
 
@@ -12,10 +13,12 @@ CONFIGS.update(HYBRID_CONFIGS)
 CONFIGS.update(ZUDISUN_CONFIGS)
 CONFIGS.update(FUGEVIK_CONFIGS)
 CONFIGS.update(VABEDRA_CONFIGS)
+CONFIGS.update(FIRONEX_CONFIGS)
 
 __all__ = ["LlamaConfig", "LlamaForCausalLM", "ReperaxConfig",
            "ReperaxForCausalLM", "ZudisunConfig",
            "ZudisunForCausalLM", "FugevikConfig", "FugevikForCausalLM",
            "VabedraConfig", "VabedraForCausalLM",
+           "FironexConfig", "FironexForCausalLM",
            "CONFIGS", "architecture_of", "build_model",
            "load_model", "register_architecture"]

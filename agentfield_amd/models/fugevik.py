@@ -56,6 +56,11 @@ class LatentAttnSpec:
     window: int = 0             # 0: every earlier key
     rot_dims: int = 0           # leading dims of the rotary part that turn
     rot_base: float = 10000.0
+    rot_scaling: dict | None = None
+    rot_pairs: bool = True      # dim 2i turns with 2i+1; False: i with i+half
+    gate: str = "element"       # output gate per "element" or per "head"
+    sink: bool = True           # learned per-head term in the denominator
+    kv_from: int | None = None  # layer whose latents and key parts are used
 
 
 @dataclass
@@ -211,6 +216,16 @@ def _pad8(n: int) -> int:
     return n + (-n) % 8
 
 
+def pad_rows(parts) -> torch.Tensor:
+    """Stack row blocks, each padded with zeros to a multiple of 8 rows."""
+    rows = []
+    for t in parts:
+        rows.append(t)
+        if t.shape[0] % 8:
+            rows.append(t.new_zeros(8 - t.shape[0] % 8, t.shape[1]))
+    return torch.cat(rows, 0)
+
+
 # ----------------------------------------------------------------- mixers
 class LatentAttention(nn.Module):
     """[q | latent, rotary key part | gate logits] = W h (one GEMM).  The
@@ -218,7 +233,9 @@ class LatentAttention(nn.Module):
     W_uv,h c.  Since q_u . (W_uk,h c) = (q_u W_uk,h) . c and sum_j w_j
     W_uv,h c_j = W_uv,h sum_j w_j c_j, attention runs over the cached rows
     [c | rot(key part)] directly (ops.masked_attention, one K/V head, values
-    inside the key rows) between two per-head batched GEMMs."""
+    inside the key rows) between two per-head batched GEMMs.  A layer with
+    `kv_from` has no down projection: it reads that layer's pages, which hold
+    this step's rows by the time it runs, through its own W_uk and W_uv."""
 
     def __init__(self, spec: LatentAttnSpec, width: int, eps: float):
         super().__init__()
@@ -226,26 +243,35 @@ class LatentAttention(nn.Module):
         self.eps = eps
         self.nq = s.heads * (s.dim + s.rot_dim)
         self.nc = s.kv_rank + s.rot_dim
-        self.ng = s.heads * s.vdim
+        self.ng = s.heads * (s.vdim if s.gate == "element" else 1)
         # blocks start at multiples of 8 rows so every view is 16-byte aligned
         self.c0 = _pad8(self.nq)
-        self.g0 = self.c0 + _pad8(self.nc)
+        self.g0 = self.c0 + (_pad8(self.nc) if s.kv_from is None else 0)
         self.w_in = nn.Parameter(torch.empty(self.g0 + _pad8(self.ng), width))
-        self.c_norm = nn.Parameter(torch.empty(s.kv_rank))
+        self.c_norm = nn.Parameter(torch.empty(s.kv_rank)) \
+            if s.kv_from is None else None
         self.uk = nn.Parameter(torch.empty(s.heads, s.dim, s.kv_rank))
         self.uv = nn.Parameter(torch.empty(s.heads, s.kv_rank, s.vdim))
         self.o = nn.Parameter(torch.empty(width, s.heads * s.vdim))
-        self.register_buffer("sink", _f32(s.heads))
+        self.register_buffer("sink", _f32(s.heads) if s.sink else None)
         self.register_buffer(
-            "inv_freq", sm.rotary_inv_freq(s.rot_dims, s.rot_base, "cpu")
+            "inv_freq", sm.scaled_inv_freq(s.rot_dims, s.rot_base,
+                                           s.rot_scaling)
             if s.rot_dims > 0 else None)
 
-    def forward(self, h, cache: HybridCache, run: int, md, positions):
+    def forward(self, h, cache: HybridCache, run: int, md, positions,
+                ctx: dict | None = None):
         s = self.spec
         T = h.shape[0]
         p = sm.matmul(h, self.w_in)
         q = p[:, :self.nq]
-        dkv = p[:, self.c0:self.c0 + self.nc]
+        own = s.kv_from is None
+        dkv = p[:, self.c0:self.c0 + self.nc] if own else None
+        pages = cache.k[run if own else s.kv_from]
+        tab = None
+        if self.inv_freq is not None:
+            tab = sm.step_rotary(ctx, positions, self.inv_freq, s.rot_dims,
+                                 s.rot_base, s.rot_scaling)
         g = p[:, self.g0:self.g0 + self.ng]
         qu = q.view(T, s.heads, s.dim + s.rot_dim)[:, :, :s.dim]
         # attention queries per head [q in latent space | rotated part]: the
@@ -254,14 +280,33 @@ class LatentAttention(nn.Module):
         torch.bmm(qu.transpose(0, 1), self.uk,
                   out=qf.view(T, s.heads, self.nc)[:, :, :s.kv_rank]
                   .transpose(0, 1))
-        sm.latent_prep(q, dkv, qf, self.c_norm, self.eps, self.inv_freq,
-                       positions, cache.k[run], md.slots, s.heads, s.dim)
-        ol = sm.masked_attention(qf, cache.k[run], None, md, positions,
-                                 s.scale, s.heads, window=s.window,
+        sm.latent_prep(q, dkv, qf, self.c_norm, self.eps, None, positions,
+                       pages, md.slots, s.heads, s.dim, rot_tab=tab,
+                       pairs=s.rot_pairs)
+        ol = sm.masked_attention(qf, pages, None, md, positions, s.scale,
+                                 s.heads, window=s.window,
                                  sink=self.sink, v_width=s.kv_rank)
         ov = torch.bmm(ol.view(T, s.heads, s.kv_rank).transpose(0, 1),
                        self.uv)                              # [H, T, vdim]
         return sm.matmul(sm.gate_heads(ov, g), self.o)
+
+
+    def load(self, get: Callable[[str], torch.Tensor], pre: str):
+        """Projections and latent norm from checkpoint tensors '<pre>q|dkv|
+        dkv.norm|uk|uv|g|o'; linear weights are [out, in], head by head."""
+        s = self.spec
+
+        def put(dst, src):
+            dst.copy_(src.to(dst.device, dst.dtype))
+        own = s.kv_from is None
+        put(self.w_in, pad_rows([get(pre + n) for n in
+                                 (("q", "dkv", "g") if own else ("q", "g"))]))
+        if own:
+            put(self.c_norm, get(pre + "dkv.norm"))
+        put(self.uk, get(pre + "uk").view(s.heads, s.dim, s.kv_rank))
+        put(self.uv, get(pre + "uv").view(s.heads, s.vdim, s.kv_rank)
+            .transpose(1, 2))
+        put(self.o, get(pre + "o"))
 
 
 class BiasedAttention(nn.Module):
@@ -283,7 +328,8 @@ class BiasedAttention(nn.Module):
         self.register_buffer("r1", _f32(s.heads))
         self.register_buffer("r2", _f32(s.heads))
 
-    def forward(self, h, cache: HybridCache, run: int, md, positions):
+    def forward(self, h, cache: HybridCache, run: int, md, positions,
+                ctx: dict | None = None):
         s = self.spec
         p = sm.matmul(h, self.w_in)
         q = p[:, :self.nq]
@@ -389,12 +435,13 @@ class FugevikForCausalLM(nn.Module):
         # a sublayer's output enters the streams in the same kernel that
         # reads the next sublayer's input out of them
         back = (None, None, None)
+        ctx: dict = {}          # what the layers of one step share
         for run, L in enumerate(self.layers):
             port = L.port1
             h = sm.hyper_conv_step(x, *back, port.inw, port.norm, eps,
                                    port.canon, cache.state["canon1"][run], md,
                                    positions, dt)
-            y = L.mixer(h, cache, run, md, positions)
+            y = L.mixer(h, cache, run, md, positions, ctx)
             back = (y, port.mix, port.outw)
             if L.mlp is not None:
                 port = L.port2
@@ -422,15 +469,6 @@ class FugevikForCausalLM(nn.Module):
         def put(dst, src):
             dst.copy_(src.to(dst.device, dst.dtype))
 
-        def blocks(dst, parts):
-            """Stack row blocks, each padded to a multiple of 8 rows."""
-            rows = []
-            for t in parts:
-                rows.append(t)
-                if t.shape[0] % 8:
-                    rows.append(t.new_zeros(8 - t.shape[0] % 8, t.shape[1]))
-            put(dst, torch.cat(rows, 0))
-
         def port(pt, pre, q):
             put(pt.norm, get(f"{pre}norm{q}"))
             put(pt.canon, get(f"{pre}canon{q}"))
@@ -444,20 +482,16 @@ class FugevikForCausalLM(nn.Module):
             port(L.port1, pre, 1)
             m, s = L.mixer, L.mixer.spec
             if isinstance(m, LatentAttention):
-                blocks(m.w_in, [get(mp + "q"), get(mp + "dkv"), get(mp + "g")])
-                put(m.c_norm, get(mp + "dkv.norm"))
-                put(m.uk, get(mp + "uk").view(s.heads, s.dim, s.kv_rank))
-                put(m.uv, get(mp + "uv").view(s.heads, s.vdim, s.kv_rank)
-                    .transpose(1, 2))
+                m.load(get, mp)
                 put(m.sink, get(mp + "sink"))
             else:
                 parts = [get(mp + "q")]
                 if s.kv_from is None:
                     parts += [get(mp + "k"), get(mp + "v")]
-                blocks(m.w_in, parts)
+                put(m.w_in, pad_rows(parts))
                 put(m.r1, get(mp + "r1"))
                 put(m.r2, get(mp + "r2"))
-            put(m.o, get(mp + "o"))
+                put(m.o, get(mp + "o"))
             if L.mlp is not None:
                 port(L.port2, pre, 2)
                 put(L.mlp.up, get(pre + "mlp.up"))

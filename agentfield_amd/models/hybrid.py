@@ -220,7 +220,8 @@ class HybridCache:
 
       "kv":    (kv_heads, dk, dv) or None - K/V pages [P, G, page, dk] /
                [P, G, page, dv] in the model dtype (dv 0: key pages only,
-               for layers whose values are part of the key rows)
+               for layers whose values are part of the key rows; kv_heads may
+               be a pair (key heads, value heads))
       "state": {name: (shape, "f32" | "model")} - per-sequence tensors
                [slots, *shape] (recurrent matrices, token-shift rows,
                convolution inputs, ...)
@@ -240,11 +241,11 @@ class HybridCache:
         for r, need in enumerate(layout):
             kv = need.get("kv")
             if kv is not None:
-                G, dk, dv = kv
+                G, Gv, dk, dv = self._heads(kv)
                 self.k[r] = torch.zeros(num_pages, G, page_size, dk,
                                         dtype=dtype, device=device)
                 if dv > 0:
-                    self.v[r] = torch.zeros(num_pages, G, page_size, dv,
+                    self.v[r] = torch.zeros(num_pages, Gv, page_size, dv,
                                             dtype=dtype, device=device)
             for name, (shape, kind) in (need.get("state") or {}).items():
                 self.state.setdefault(name, {})[r] = torch.zeros(
@@ -254,12 +255,18 @@ class HybridCache:
         self.shift = self.state.get("shift", {})
 
     @staticmethod
+    def _heads(kv):
+        """(key heads, value heads, dk, dv) of a layout's "kv" entry."""
+        G, dk, dv = kv
+        return (*G, dk, dv) if isinstance(G, tuple) else (G, G, dk, dv)
+
+    @staticmethod
     def bytes_per_page(layout: list, page_size: int, itemsize: int = 2) -> int:
         n = 0
         for need in layout:
             if need.get("kv") is not None:
-                G, dk, dv = need["kv"]
-                n += G * page_size * (dk + dv) * itemsize
+                G, Gv, dk, dv = HybridCache._heads(need["kv"])
+                n += page_size * (G * dk + Gv * dv) * itemsize
         return max(n, 1)
 
     @staticmethod

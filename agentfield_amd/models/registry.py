@@ -91,9 +91,16 @@ def _load_vabedra(path, device="cpu", dtype=None, **kw):
                         max_position=kw.get("max_position"))
 
 
+def _load_fironex(path, device="cpu", dtype=None, **kw):
+    from .fironex import load_fironex
+    return load_fironex(path, device=device, dtype=dtype,
+                        max_position=kw.get("max_position"))
+
+
 register_architecture(["LlamaForCausalLM", "MistralForCausalLM",
                        "MixtralForCausalLM"], _load_llama)
 register_architecture("Reperax", _load_reperax)
 register_architecture("Zudisun", _load_zudisun)
 register_architecture("Fugevik", _load_fugevik)
 register_architecture("Vabedra", _load_vabedra)
+register_architecture("Fironex", _load_fironex)

@@ -329,11 +329,8 @@ class SinkWindowAttention(nn.Module):
         tab = None
         if self.inv_freq is not None:
             # layers that rotate alike share the step's cos / sin table
-            key = (s.rot_dims, s.rot_base,
-                   tuple(sorted((s.rot_scaling or {}).items())))
-            tab = ctx.get(key)
-            if tab is None:
-                tab = ctx[key] = sm.rotary_table(positions, self.inv_freq)
+            tab = sm.step_rotary(ctx, positions, self.inv_freq, s.rot_dims,
+                                 s.rot_base, s.rot_scaling)
         q = sm.qk_rope_cache(
             p[:, :a], p[:, a:b], p[:, b:c], s.heads, s.kv_heads, self.eps,
             cache.k[run], cache.v[run], md.slots, positions,

@@ -131,7 +131,9 @@ def _mix_sigs() -> dict:
             "afm_dual_norm_shift": [p, p, p, p, p, p, p, p, p, p, p, p, p, f,
                                     i, i, i, p],
             "afm_scatter_state": [p, p, p, p, i, i, p],
-            "afm_norm_rows": [p, p, p, p, f, i, i, i, i, p],
+            "afm_norm_rows": [p, p, p, p, f, i, i, i, i, i, p],
+            "afm_sandwich_norm": [p, p, p, i64, i, p, p, f, f, i, i, i, p],
+            "afm_xielu": [p, p, i64, p, i, i, i, p],
             "afm_headnorm_gate": [p, p, p, p, f, i, i, i, i64, i, i, p],
             "afm_polynorm": [p, p, p, f, i, i, i64, i, p],
             "afm_gated_residual": [p, p, f, p, f, p, i64, p, p, p, i64, p,
@@ -149,20 +151,24 @@ def _mix_sigs() -> dict:
                                   i, i, i, i64, i64, i64, i, p],
             "afm_masked_attention": [p, p, p, p, p, p, p, f, i, i, i, i, i, i,
                                      i, i, i, i64, i, p, p, p, f, p, p, i64,
-                                     i, i, p],
+                                     i, i, i, p],
+            "afm_diff_combine": [p, p, p, p, i64, f, f, f, i, i, i, i, i, i,
+                                 p],
             "afm_attn_prefill_mfma": [p, p, p, p, p, p, p, p, p, f, i, i, i, i,
                                       i, i, i, i, i, i64, p, f, p, p, i64, i,
-                                      p],
+                                      i, p],
+            "afm_diff_prefill_mfma": [p, p, p, p, p, p, p, p, p, f, i, i, i, i,
+                                      i, i, i, i, i64, p, i64, f, f, f, p],
             "afm_attn_heads_mfma": [p, p, p, p, p, p, p, f, i, i, i, i, i, i,
                                     i, i, i, i64, i, p, p, p, f, p, p, i64, i,
-                                    p],
+                                    i, p],
             "afm_attn_split_combine": [p, p, p, i, i, i, i, p],
             "afm_linear_scan": [p, p, p, p, p, p, p, p, p, p, p, p, p, f, f, f,
                                 i, i, i, i, i, i64, i64, i64, i64, i, p],
         },
         "conv": {
-            "afm_causal_conv": [p, p, i64, p, p, p, p, p, p, p, i, i, i, i, i,
-                                i, p],
+            "afm_causal_conv": [p, p, i64, p, p, p, p, p, p, p, p, i, i, i, i,
+                                i, i, p],
         },
         "ssm": {
             "afm_selective_scan": [p, p, p, p, p, p, i64, p, i64, p, p, p, p,
@@ -181,17 +187,28 @@ def _mix_sigs() -> dict:
             "afm_hyper_step": [p, p, i64, p, p, p, p, f, p, i, i, i, i, p, p,
                                p, p, i, p, i, p],
             "afm_canon_conv": [p, p, p, p, p, p, p, p, i, i, i, i, i, p],
-            "afm_latent_prep": [p, p, p, i64, p, i64, p, p, p, p, f, i, i,
-                                i, i, i, i, i, p],
-            "afm_gate_heads": [p, p, p, i64, i, i, i, i, p],
             "afm_relu2": [p, p, i64, i, i, i, p],
+        },
+        "latent": {
+            "afm_latent_prep": [p, p, p, i64, p, i64, p, p, p, f, i, i, i, i,
+                                i, i, i, i, p],
+            "afm_gate_heads": [p, p, p, i64, i, i, i, i, i, p],
+        },
+        "rope": {
+            "afm_rotary_table": [p, p, p, i, i, p],
+            "afm_qk_rope_cache": [p, p, i64, p, i64, p, i64, p, p, p, p, p,
+                                  p, i, p, p, p, f, i, i, i, i, i, i, i, i, i,
+                                  p],
+        },
+        "rglru": {
+            "afm_rglru_gates": [p, p, p, p, p, p, p, p, i, i, i, i, p],
+            "afm_rglru_scan": [p, p, p, p, p, i64, p, p, p, p, i, i, i, i, p],
+            "afm_rglru_step": [p, p, p, p, i64, p, p, p, p, i64, p, p, p, p,
+                               p, p, p, p, i, i, i, i, p],
         },
         "delta": {
             "afm_delta_scan": [p, p, p, i64, p, i64, p, i64, p, i64, p, i64,
                                p, p, p, p, p, i, i, i, i, i, i, f, i, i, p],
-            "afm_rotary_table": [p, p, p, i, i, p],
-            "afm_qk_rope_cache": [p, p, i64, p, i64, p, i64, p, p, p, p, p,
-                                  p, i, p, p, p, f, i, i, i, i, i, i, i, p],
             "afm_postnorm_sum": [p, p, p, i64, i, p, i64, p, p, p, f, f, i,
                                  i, i, p],
             "afm_gate_gather": [p, p, i64, p, i64, i, p, i, i, i, p],

@@ -155,10 +155,13 @@ def dual_norm_shift(x: torch.Tensor, w1: torch.Tensor,
 
 def norm_rows(x: torch.Tensor, w: torch.Tensor, eps: float,
               rows: torch.Tensor | None, out_dtype: torch.dtype,
-              one_plus: bool = True) -> torch.Tensor:
-    """RMSNorm of selected fp32 rows: x[rows] / rms * (1 + w) (or * w)."""
+              one_plus: bool = True, center: bool = False) -> torch.Tensor:
+    """RMSNorm of selected fp32 rows: x[rows] / rms * (1 + w) (or * w);
+    center: layer norm, the row's mean taken off first."""
     if not _gpu(x):
         xs = x[rows.long()] if rows is not None else x
+        if center:
+            xs = xs - xs.mean(-1, keepdim=True)
         r = torch.rsqrt(xs.pow(2).mean(-1, keepdim=True) + eps)
         wf = w.float() + 1.0 if one_plus else w.float()
         return (xs * r * wf).to(out_dtype)
@@ -167,8 +170,8 @@ def norm_rows(x: torch.Tensor, w: torch.Tensor, eps: float,
     out = torch.empty(R, W, dtype=out_dtype, device=x.device)
     rc = _L().afm_norm_rows(_lib.ptr(out), _lib.ptr(x), _lib.ptr(w),
                             _lib.ptr(rows), float(eps), R, W,
-                            1 if one_plus else 0, _code(out),
-                            _lib.cur_stream())
+                            1 if one_plus else 0, 1 if center else 0,
+                            _code(out), _lib.cur_stream())
     _lib.check(rc, "afm_norm_rows")
     return out
 
@@ -207,6 +210,18 @@ def qk_norm_cache(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
         _lib.cur_stream())
     _lib.check(rc, "afm_qk_norm_cache")
     return out
+
+
+def _row_tiles(lens, rows: int, device):
+    """Tile map of packed chunks for the tile kernels: (tiles, sequence of
+    every tile, its first row inside the chunk)."""
+    ts, tq = [], []
+    for b, ln in enumerate(lens):
+        for q0 in range(0, ln, rows):
+            ts.append(b)
+            tq.append(q0)
+    return (len(ts), torch.tensor(ts, dtype=torch.int32, device=device),
+            torch.tensor(tq, dtype=torch.int32, device=device))
 
 
 def masked_attention(q: torch.Tensor, kcache: torch.Tensor,
@@ -273,22 +288,16 @@ def masked_attention(q: torch.Tensor, kcache: torch.Tensor,
     out = torch.empty(T, H * dv, dtype=q.dtype, device=q.device)
     lens = getattr(md, "seq_lens", None)
     extra = (_lib.ptr(sink), float(softcap), _lib.ptr(r1), _lib.ptr(r2),
-             int(ldv), int(keep_first))
+             int(ldv), int(keep_first), 1)
     if (q.dtype == torch.bfloat16 and lens is not None and dk <= 576
             and dv <= 512 and max(lens) >= MFMA_MIN_ROWS):
         # prompt portions: 64-row tiles on the matrix cores
-        ts, tq = [], []
-        for b, ln in enumerate(lens):
-            for q0 in range(0, ln, 64):
-                ts.append(b)
-                tq.append(q0)
-        tile_seq = torch.tensor(ts, dtype=torch.int32, device=q.device)
-        tile_q0 = torch.tensor(tq, dtype=torch.int32, device=q.device)
+        nt, tile_seq, tile_q0 = _row_tiles(lens, 64, q.device)
         rc = _L().afm_attn_prefill_mfma(
             _lib.ptr(out), _lib.ptr(q), _lib.ptr(kcache), _lib.ptr(vsrc),
             _lib.ptr(md.block_table), _lib.ptr(md.cu_seqlens),
             _lib.ptr(md.q_start), _lib.ptr(tile_seq), _lib.ptr(tile_q0),
-            float(scale), len(ts), H, G, dk, dv, page,
+            float(scale), nt, H, G, dk, dv, page,
             md.block_table.shape[1], int(chunk), int(window), _rowstride(q),
             *extra, _lib.cur_stream())
         if rc != 9004:          # 9004: no tile kernel for this head geometry
@@ -341,6 +350,99 @@ def masked_attention(q: torch.Tensor, kcache: torch.Tensor,
         int(chunk), int(window), _rowstride(q), nsplit, _lib.ptr(part_o),
         _lib.ptr(part_ml), *extra, _code(q), _lib.cur_stream())
     _lib.check(rc, "afm_masked_attention")
+    return out
+
+
+def diff_attention(q: torch.Tensor, kcache: torch.Tensor,
+                   vcache: torch.Tensor, md, positions: torch.Tensor,
+                   scale: float, heads: int, lam: float, diff: float,
+                   eps: float, gate: torch.Tensor | None = None,
+                   window: int = 0) -> torch.Tensor:
+    """Differential attention of packed rows over the paged cache: every head
+    has two query / key maps over the same values, each with a softmax of its
+    own (visibility as in masked_attention), a1 and a2 their outputs:
+
+        o = a1 - lam a2;  o <- o / sqrt(mean(o^2) + eps) * (1 - diff)
+
+    per head, times sigmoid(gate) per element.  q [T, 2H*dk] laid out [K/V
+    head][map][head of the group]; kcache [P, 2G, page, dk] ([K/V head][map]),
+    vcache [P, G, page, dv]; gate [T, H*dv] logits (may be a strided view) ->
+    [T, H*dv]."""
+    T = q.shape[0]
+    H = heads
+    _, G2, page, dk = kcache.shape
+    G, dv = vcache.shape[1], vcache.shape[3]
+    if G2 != 2 * G:
+        raise ValueError("diff_attention: two key heads per value head")
+    hpg = H // G
+    if not _gpu(q):
+        vv = vcache.repeat_interleave(2, dim=1)
+        a = masked_attention(q.float(), kcache, vv, md, positions, scale,
+                             2 * H, window=window)
+        a = a.view(T, G, 2, hpg, dv)
+        o = (a[:, :, 0] - lam * a[:, :, 1]).reshape(T, H, dv)
+        o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) \
+            * (1.0 - diff)
+        o = o.reshape(T, H * dv)
+        if gate is not None:
+            o = o * torch.sigmoid(gate.float())
+        return o.to(q.dtype)
+    out = torch.empty(T, H * dv, dtype=q.dtype, device=q.device)
+    lens = getattr(md, "seq_lens", None)
+    maxp = md.block_table.shape[1]
+    ldg = _rowstride(gate) if gate is not None else 0
+    if (q.dtype == torch.bfloat16 and lens is not None and dk <= 128
+            and dv <= 256 and max(lens) >= MFMA_MIN_ROWS):
+        # prompt portions: both maps of a head in one workgroup, combined,
+        # normed and gated before they leave it
+        nt, tile_seq, tile_q0 = _row_tiles(lens, 64, q.device)
+        rc = _L().afm_diff_prefill_mfma(
+            _lib.ptr(out), _lib.ptr(q), _lib.ptr(kcache), _lib.ptr(vcache),
+            _lib.ptr(md.block_table), _lib.ptr(md.cu_seqlens),
+            _lib.ptr(md.q_start), _lib.ptr(tile_seq), _lib.ptr(tile_q0),
+            float(scale), nt, H, G, dk, dv, page, maxp, int(window),
+            _rowstride(q), _lib.ptr(gate), ldg, float(lam), float(diff),
+            float(eps), _lib.cur_stream())
+        if rc != 9004:
+            _lib.check(rc, "afm_diff_prefill_mfma")
+            return out
+    # rows of their own: partial softmaxes of all maps, merged, combined,
+    # normed and gated by one wave per (row, head)
+    reach = min(x for x in (window, maxp * page) if x > 0)
+    heads_tile = (q.dtype == torch.bfloat16 and hpg >= HEADS_MFMA_MIN
+                  and dk <= 576 and dv <= 512)
+    if heads_tile:
+        wgs = T * G2 * -(-hpg // 16)
+        nsplit = max(1, min(16, 2048 // max(1, wgs), -(-reach // 64)))
+    else:
+        wgs = T * G2 * -(-hpg // min(8, hpg))
+        nsplit = max(1, min(8, 2048 // max(1, wgs), reach // 128))
+        if max(dk, dv) > 64 * (16 // q.element_size()):
+            nsplit = 1          # the kernel for such wide heads has no splits
+    part_o = torch.empty(T, 2 * H, nsplit, dv, dtype=torch.float32,
+                         device=q.device)
+    part_ml = torch.empty(T, 2 * H, nsplit, 2, dtype=torch.float32,
+                          device=q.device)
+    extra = (None, 0.0, None, None, dv, 0, 2)
+    common = (_lib.ptr(q), _lib.ptr(kcache), _lib.ptr(vcache),
+              _lib.ptr(md.block_table), _lib.ptr(md.row_seq),
+              _lib.ptr(positions), float(scale), T, 2 * H, G2, dk, dv, page,
+              maxp, 0, int(window), _rowstride(q), nsplit, _lib.ptr(part_o),
+              _lib.ptr(part_ml), *extra)
+    rc = 9004
+    if heads_tile:
+        rc = _L().afm_attn_heads_mfma(None, *common, _lib.cur_stream())
+        if rc != 9004:
+            _lib.check(rc, "afm_attn_heads_mfma")
+    if rc == 9004:
+        rc = _L().afm_masked_attention(None, *common, _code(q),
+                                       _lib.cur_stream())
+        _lib.check(rc, "afm_masked_attention")
+    rc = _L().afm_diff_combine(
+        _lib.ptr(out), _lib.ptr(part_o), _lib.ptr(part_ml), _lib.ptr(gate),
+        ldg, float(lam), float(diff), float(eps), T, H, hpg, nsplit, dv,
+        _code(q), _lib.cur_stream())
+    _lib.check(rc, "afm_diff_combine")
     return out
 
 
@@ -706,13 +808,14 @@ def moe_combine(ys: torch.Tensor, pos: torch.Tensor, weights: torch.Tensor,
 
 # ------------------------------------------------- selective state space
 def causal_conv(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None,
-                state: torch.Tensor, md, silu: bool = True) -> torch.Tensor:
+                state: torch.Tensor, md, silu: bool = True,
+                in_bias: torch.Tensor | None = None) -> torch.Tensor:
     """Depthwise causal convolution over packed chunks: out[t, c] = act(b[c]
-    + sum_j w[j, c] x[t - (taps-1-j), c]); w is tap-major [taps, C], its last
-    row weighing the current token.  Inputs from before a chunk come from the sequence's slot
+    + sum_j w[j, c] (x[t - (taps-1-j), c] + in_bias[c])); w is tap-major
+    [taps, C], its last row weighing the current token.  Inputs from before a chunk come from the sequence's slot
     of `state` [slots, taps-1, C] (storage dtype, oldest first), inputs
-    before position 0 are zero; afterwards the slot holds the sequence's last
-    taps-1 inputs.  x [T, C] may be a strided view."""
+    before position 0 are zero (in_bias included); afterwards the slot holds
+    the sequence's last taps-1 inputs x.  x [T, C] may be a strided view."""
     T, C = x.shape
     taps = w.shape[0]
     B = md.q_start.numel()
@@ -731,8 +834,12 @@ def causal_conv(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None,
             acc = torch.zeros(r1 - r0, C)
             if bias is not None:
                 acc += bias.float()
+            inp = cat
+            if in_bias is not None:     # nothing is added before position 0
+                inp = cat + in_bias.float()
+                inp[:max(0, taps - 1 - qs[b])] = 0.0
             for j in range(taps):
-                acc += wf[j] * cat[j:j + r1 - r0]
+                acc += wf[j] * inp[j:j + r1 - r0]
             out[r0:r1] = acc
             if taps > 1:
                 state[sl[b]][:taps - 1] = cat[-(taps - 1):].to(state.dtype)
@@ -742,8 +849,8 @@ def causal_conv(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None,
     out = torch.empty(T, C, dtype=x.dtype, device=x.device)
     rc = _L().afm_causal_conv(
         _lib.ptr(out), _lib.ptr(x), _rowstride(x), _lib.ptr(w),
-        _lib.ptr(bias), _lib.ptr(state), _lib.ptr(md.row_seq),
-        _lib.ptr(md.cu_seqlens), _lib.ptr(md.q_start),
+        _lib.ptr(bias), _lib.ptr(in_bias), _lib.ptr(state),
+        _lib.ptr(md.row_seq), _lib.ptr(md.cu_seqlens), _lib.ptr(md.q_start),
         _lib.ptr(md.state_slots), T, B, C, taps, 1 if silu else 0, _code(x),
         _lib.cur_stream())
     _lib.check(rc, "afm_causal_conv")
@@ -1082,79 +1189,89 @@ def canon_conv(n: torch.Tensor, w: torch.Tensor, state: torch.Tensor, md,
     return h
 
 
-def rotate_pairs(x: torch.Tensor, positions: torch.Tensor,
-                 inv_freq: torch.Tensor) -> torch.Tensor:
-    """Interleaved rotary embedding of the leading 2*len(inv_freq) elements
-    of the last axis (element 2i pairs with 2i+1; angle = position * f_i);
-    x [T, ..., d] fp32, CPU helper of latent_prep."""
-    r = 2 * inv_freq.numel()
-    ang = positions.float()[:, None] * inv_freq.float()[None]
-    shape = [x.shape[0]] + [1] * (x.dim() - 2) + [r // 2]
-    c, s = ang.cos().view(shape), ang.sin().view(shape)
-    u, v = x[..., 0:r:2], x[..., 1:r:2]
+def rotate_rows(x: torch.Tensor, tab: torch.Tensor,
+                pairs: bool) -> torch.Tensor:
+    """Rotary embedding of the leading tab.shape[1] elements of the last axis
+    by the rows' rotary_table: element 2i with 2i+1 (pairs) or element i with
+    i + half; x [T, ..., d] fp32 (CPU form of what the row kernels do)."""
+    half = tab.shape[1] // 2
+    shape = [x.shape[0]] + [1] * (x.dim() - 2) + [half]
+    c, s = tab[:, :half].reshape(shape), tab[:, half:].reshape(shape)
+    first = slice(0, 2 * half, 2) if pairs else slice(0, half)
+    second = slice(1, 2 * half, 2) if pairs else slice(half, 2 * half)
+    u, v = x[..., first], x[..., second]
     out = x.clone()
-    out[..., 0:r:2] = u * c - v * s
-    out[..., 1:r:2] = v * c + u * s
+    out[..., first] = u * c - v * s
+    out[..., second] = v * c + u * s
     return out
 
 
-def latent_prep(q: torch.Tensor, dkv: torch.Tensor, qf: torch.Tensor,
-                norm_w: torch.Tensor, eps: float,
+def latent_prep(q: torch.Tensor, dkv: torch.Tensor | None, qf: torch.Tensor,
+                norm_w: torch.Tensor | None, eps: float,
                 inv_freq: torch.Tensor | None, positions: torch.Tensor,
                 kcache: torch.Tensor, slots: torch.Tensor, heads: int,
-                dim: int) -> torch.Tensor:
+                dim: int, rot_tab: torch.Tensor | None = None,
+                pairs: bool = True) -> torch.Tensor:
     """Row steps of latent attention.  dkv [T, R + rd] (may be a strided
     view) holds the latent and one rotary key part: the latent is RMS-normed
-    with a plain weight, the key part rotated (interleaved pairs on its first
-    2*len(inv_freq) elements), and [latent | key part] is appended to the key
-    pages kcache [P, 1, page, R + rd] at `slots`.  q [T, H*(dim + rd)] holds
-    per head [unrotated | rotary part].  qf [T, H*(R + rd)] are the attention
-    queries, per head [unrotated part carried into latent space | rotated
-    rotary part]: the caller has filled the first R elements of every head,
-    the rotary slices are written here.  Returns qf."""
+    with a plain weight, the key part rotated (its first 2*len(inv_freq)
+    elements; pairs: element 2i with 2i+1, otherwise i with i + len(inv_freq);
+    rot_tab gives the rows' ready rotary_table), and [latent | key part] is
+    appended to the key pages kcache [P, 1, page, R + rd] at `slots`.  dkv
+    None: no key row (the layer reads another layer's pages).  q [T, H*(dim +
+    rd)] holds per head [unrotated | rotary part].  qf [T, H*(R + rd)] are the
+    attention queries, per head [unrotated part carried into latent space |
+    rotated rotary part]: the caller has filled the first R elements of every
+    head, the rotary slices are written here.  Returns qf."""
     T = q.shape[0]
     H = heads
-    R = norm_w.numel()
-    rd = dkv.shape[1] - R
-    dkc = R + rd
-    page = kcache.shape[2]
-    rot = 2 * inv_freq.numel() if inv_freq is not None else 0
+    page, dkc = kcache.shape[2], kcache.shape[3]
+    rd = q.shape[1] // H - dim
+    R = dkc - rd
+    if rot_tab is None and inv_freq is not None and inv_freq.numel() > 0:
+        rot_tab = rotary_table(positions, inv_freq.double())
+    rot = rot_tab.shape[1] if rot_tab is not None else 0
     if not _gpu(q):
+        qr = q.float().view(T, H, dim + rd)[..., dim:]
+        if rot:
+            qr = rotate_rows(qr, rot_tab, pairs)
+        qf.view(T, H, dkc)[..., R:] = qr.to(qf.dtype)
+        if dkv is None:
+            return qf
         d = dkv.float()
         c = d[:, :R] * torch.rsqrt(d[:, :R].pow(2).mean(-1, keepdim=True)
                                    + eps) * norm_w.float()
-        kr = d[:, R:]
-        qr = q.float().view(T, H, dim + rd)[..., dim:]
-        if rot:
-            kr = rotate_pairs(kr, positions, inv_freq)
-            qr = rotate_pairs(qr, positions, inv_freq)
+        kr = rotate_rows(d[:, R:], rot_tab, pairs) if rot else d[:, R:]
         pg = torch.div(slots, page, rounding_mode="floor")
         off = slots - pg * page
         kcache[pg, 0, off] = torch.cat([c, kr], 1).to(kcache.dtype)
-        qf.view(T, H, dkc)[..., R:] = qr.to(qf.dtype)
         return qf
     assert qf.is_contiguous() and qf.shape == (T, H * dkc)
     rc = _L().afm_latent_prep(
         _lib.ptr(qf), _lib.ptr(kcache), _lib.ptr(q), _rowstride(q),
-        _lib.ptr(dkv), _rowstride(dkv), _lib.ptr(norm_w),
-        _lib.ptr(inv_freq), _lib.ptr(positions), _lib.ptr(slots), float(eps),
-        T, H, dim, rd, R, rot, _code(q), _lib.cur_stream())
+        _lib.ptr(dkv), _rowstride(dkv) if dkv is not None else 0,
+        _lib.ptr(norm_w), _lib.ptr(rot_tab), _lib.ptr(slots), float(eps), T,
+        H, dim, rd, R, rot, 1 if pairs else 0, _code(q), _lib.cur_stream())
     _lib.check(rc, "afm_latent_prep")
     return qf
 
 
 def gate_heads(o: torch.Tensor, gate: torch.Tensor) -> torch.Tensor:
-    """out[t, h*dv + d] = o[h, t, d] * sigmoid(gate[t, h*dv + d]): per-head
-    results [H, T, dv] back to token rows, times an element-wise output gate
-    (logits [T, H*dv], may be a strided view)."""
+    """Per-head results [H, T, dv] back to token rows [T, H*dv], times the
+    sigmoid of an output gate: one logit per element (gate [T, H*dv]) or one
+    per head (gate [T, H]); may be a strided view."""
     H, T, dv = o.shape
+    per_head = gate.shape[1] == H
     if not _gpu(o):
-        return (o.float().transpose(0, 1).reshape(T, H * dv)
-                * torch.sigmoid(gate.float())).to(o.dtype)
+        g = torch.sigmoid(gate.float())
+        r = o.float().transpose(0, 1)
+        r = r * (g[:, :, None] if per_head else g.view(T, H, dv))
+        return r.reshape(T, H * dv).to(o.dtype)
     o = o.contiguous()
     out = torch.empty(T, H * dv, dtype=o.dtype, device=o.device)
     rc = _L().afm_gate_heads(_lib.ptr(out), _lib.ptr(o), _lib.ptr(gate),
-                             _rowstride(gate), T, H, dv, _code(o),
+                             _rowstride(gate), T, H, dv,
+                             1 if per_head else 0, _code(o),
                              _lib.cur_stream())
     _lib.check(rc, "afm_gate_heads")
     return out
@@ -1220,6 +1337,20 @@ def rotary_table(positions: torch.Tensor,
     return tab
 
 
+def step_rotary(ctx: dict | None, positions: torch.Tensor,
+                inv_freq: torch.Tensor, dims: int, base: float,
+                scaling: dict | None) -> torch.Tensor:
+    """The step's rotary_table for these frequencies, made once: `ctx` is a
+    dict that lives for one forward pass (None: nothing is shared)."""
+    if ctx is None:
+        return rotary_table(positions, inv_freq)
+    key = (dims, base, tuple(sorted((scaling or {}).items())))
+    tab = ctx.get(key)
+    if tab is None:
+        tab = ctx[key] = rotary_table(positions, inv_freq)
+    return tab
+
+
 def qk_rope_cache(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
                   heads: int, kv_heads: int, eps: float,
                   kcache: torch.Tensor, vcache: torch.Tensor,
@@ -1230,19 +1361,22 @@ def qk_rope_cache(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
                   q_norm: torch.Tensor | None = None,
                   k_norm: torch.Tensor | None = None,
                   inv_freq: torch.Tensor | None = None,
-                  rot_tab: torch.Tensor | None = None) -> torch.Tensor:
+                  rot_tab: torch.Tensor | None = None,
+                  pairs: bool = False) -> torch.Tensor:
     """Row steps in front of rotary attention.  q [T, H*dk], k [T, G*dk], v
-    [T, G*dv] (strided views allowed) get their biases; every q and k head
+    [T, Gv*dv] (strided views allowed; Gv, the value pages' heads, may be
+    fewer than G) get their biases; every q and k head
     is RMS-normed over dk with a plain weight [dk] shared by heads (skipped
     without one); the first 2*len(inv_freq) dims of each head are rotated,
-    dim i paired with i + len(inv_freq), by the angle position * f_i
+    dim i paired with i + len(inv_freq) (pairs: dim 2i with 2i + 1), by the
+    angle position * f_i
     (inv_freq float64; product, sine and cosine in double precision; or the
     rows' ready rotary_table as rot_tab); k and v are appended to the paged
     caches at `slots`.  Returns q, contiguous [T, H*dk]."""
     T = q.shape[0]
-    H, G = heads, kv_heads
+    H, G, Gv = heads, kv_heads, vcache.shape[1]
     dk = q.shape[1] // H
-    dv = v.shape[1] // G
+    dv = v.shape[1] // Gv
     page = kcache.shape[2]
     if rot_tab is None and inv_freq is not None and inv_freq.numel() > 0:
         rot_tab = rotary_table(positions, inv_freq)
@@ -1265,17 +1399,12 @@ def qk_rope_cache(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
             kf = kf * torch.rsqrt(kf.pow(2).mean(-1, keepdim=True) + eps) \
                 * k_norm.float()
         if half:
-            c, s = rot_tab[:, None, :half], rot_tab[:, None, half:]
-
-            def rot(x):
-                u, w = x[..., :half], x[..., half:2 * half]
-                return torch.cat([u * c - w * s, w * c + u * s,
-                                  x[..., 2 * half:]], -1)
-            qf, kf = rot(qf), rot(kf)
+            qf = rotate_rows(qf, rot_tab, pairs)
+            kf = rotate_rows(kf, rot_tab, pairs)
         pg = torch.div(slots, page, rounding_mode="floor")
         off = slots - pg * page
         kcache[pg, :, off] = kf.to(kcache.dtype)
-        vcache[pg, :, off] = vf.reshape(T, G, dv).to(vcache.dtype)
+        vcache[pg, :, off] = vf.reshape(T, Gv, dv).to(vcache.dtype)
         return qf.reshape(T, H * dk).to(q.dtype)
     out = torch.empty(T, H * dk, dtype=q.dtype, device=q.device)
     rc = _L().afm_qk_rope_cache(
@@ -1283,8 +1412,8 @@ def qk_rope_cache(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
         _lib.ptr(v), _rowstride(v), _lib.ptr(q_bias), _lib.ptr(k_bias),
         _lib.ptr(v_bias), _lib.ptr(q_norm), _lib.ptr(k_norm),
         _lib.ptr(rot_tab), 2 * half, _lib.ptr(kcache), _lib.ptr(vcache),
-        _lib.ptr(slots), float(eps), T, H, G, dk, dv, page, _code(q),
-        _lib.cur_stream())
+        _lib.ptr(slots), float(eps), T, H, G, Gv, dk, dv, page,
+        1 if pairs else 0, _code(q), _lib.cur_stream())
     _lib.check(rc, "afm_qk_rope_cache")
     return out
 
@@ -1418,4 +1547,131 @@ def gate_gather(z: torch.Tensor, table: torch.Tensor, ids: torch.Tensor,
                               _lib.ptr(ids), T, C, _code(z),
                               _lib.cur_stream())
     _lib.check(rc, "afm_gate_gather")
+    return out
+
+
+# =====================================================================
+# Ops of decoders with layer norms on both sides of every sublayer: the
+# norm pair around a residual add, real-gated linear recurrent units, the
+# xIELU activation (differential attention sits beside masked_attention).
+# =====================================================================
+def sandwich_norm(x: torch.Tensor, y: torch.Tensor | None, mult: float,
+                  w_post: torch.Tensor | None, w_pre: torch.Tensor | None,
+                  eps: float, dtype: torch.dtype) -> torch.Tensor | None:
+    """Layer norms on both sides of a sublayer boundary, in place on the fp32
+    residual: with y (a sublayer's output, [T, W] in the storage dtype or
+    fp32) x += mult * LN(y) * w_post; with w_pre the next sublayer's input
+    LN(x) * w_pre is returned in `dtype`."""
+    T, W = x.shape
+    if not _gpu(x):
+        def ln(u, w):
+            d = u - u.mean(-1, keepdim=True)
+            return d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) \
+                * w.float()
+        if y is not None:
+            x += mult * ln(y.float(), w_post)
+        return ln(x, w_pre).to(dtype) if w_pre is not None else None
+    h = torch.empty(T, W, dtype=dtype, device=x.device) \
+        if w_pre is not None else None
+    ref = w_pre if w_pre is not None else w_post
+    rc = _L().afm_sandwich_norm(
+        _lib.ptr(x), _lib.ptr(h), _lib.ptr(y),
+        _rowstride(y) if y is not None else 0,
+        1 if y is not None and y.dtype == torch.float32 else 0,
+        _lib.ptr(w_post), _lib.ptr(w_pre), float(mult), float(eps), T, W,
+        _code(ref), _lib.cur_stream())
+    _lib.check(rc, "afm_sandwich_norm")
+    return h
+
+
+def xielu(z: torch.Tensor, coef: torch.Tensor) -> torch.Tensor:
+    """Element-wise: z > 0: coef[0] z^2 + z / 2; z <= 0: coef[1] (e^z - 1 -
+    z) + z / 2.  coef [2] fp32; z [T, F] may be a strided view."""
+    T, F = z.shape
+    if not _gpu(z):
+        zf = z.float()
+        n = zf.clamp(max=0.0)
+        return (torch.where(zf > 0, coef[0] * zf * zf,
+                            coef[1] * (torch.expm1(n) - n))
+                + 0.5 * zf).to(z.dtype)
+    out = torch.empty(T, F, dtype=z.dtype, device=z.device)
+    rc = _L().afm_xielu(_lib.ptr(out), _lib.ptr(z), _rowstride(z),
+                        _lib.ptr(coef), T, F, _code(z), _lib.cur_stream())
+    _lib.check(rc, "afm_xielu")
+    return out
+
+
+def rglru(x: torch.Tensor, x_bias: torch.Tensor | None, y: torch.Tensor,
+          y_bias: torch.Tensor | None, conv: torch.Tensor,
+          conv_b: torch.Tensor | None, wr: torch.Tensor, br: torch.Tensor,
+          wi: torch.Tensor, bi: torch.Tensor, rate: torch.Tensor,
+          state: torch.Tensor, conv_state: torch.Tensor, md) -> torch.Tensor:
+    """Real-gated linear recurrent unit over packed chunks:
+
+        u = causal_conv(x + x_bias)            (conv tap-major [taps, C])
+        r, i = sigmoid(W u + b) per block      (wr, wi [blocks, n, n], [out, in])
+        log a = rate * r
+        S <- a S + sqrt(1 - a^2) i u;  out = S * gelu_tanh(y + y_bias)
+
+    x, y [T, C] may be strided views; br, bi, rate [C] fp32.  S lives in
+    `state` [slots, C] fp32: zero where a chunk starts at position 0, written
+    after the chunk's last row; the convolution's inputs in conv_state (see
+    causal_conv)."""
+    T, C = x.shape
+    blocks, n, _ = wr.shape
+    B = md.q_start.numel()
+    if _gpu(x) and x.dtype == torch.bfloat16 \
+            and not getattr(md, "is_prefill", True):
+        # one row per sequence: everything in one kernel
+        out = torch.empty(T, C, dtype=x.dtype, device=x.device)
+        rc = _L().afm_rglru_step(
+            _lib.ptr(out), _lib.ptr(state), _lib.ptr(conv_state), _lib.ptr(x),
+            _rowstride(x), _lib.ptr(x_bias), _lib.ptr(conv), _lib.ptr(conv_b),
+            _lib.ptr(y), _rowstride(y), _lib.ptr(y_bias), _lib.ptr(wr),
+            _lib.ptr(br), _lib.ptr(wi), _lib.ptr(bi), _lib.ptr(rate),
+            _lib.ptr(md.q_start), _lib.ptr(md.state_slots), T, C, blocks,
+            conv.shape[0], _lib.cur_stream())
+        if rc != 9004:          # 9004: a block does not fit in LDS
+            _lib.check(rc, "afm_rglru_step")
+            return out
+    u = causal_conv(x, conv, conv_b, conv_state, md, silu=False,
+                    in_bias=x_bias)
+    if not _gpu(x):
+        uf = u.float()
+        ub = uf.view(T, blocks, n)
+        zr = torch.einsum("tbk,bnk->tbn", ub, wr.float()).reshape(T, C)
+        zi = torch.einsum("tbk,bnk->tbn", ub, wi.float()).reshape(T, C)
+        log_a = rate * torch.sigmoid(zr + br)
+        a = torch.exp(log_a)
+        g = torch.sqrt(-torch.expm1(2.0 * log_a)) * torch.sigmoid(zi + bi) * uf
+        yf = y.float()
+        if y_bias is not None:
+            yf = yf + y_bias.float()
+        out = torch.empty(T, C, dtype=torch.float32)
+        cu, qs, sl = (md.cu_seqlens.tolist(), md.q_start.tolist(),
+                      md.state_slots.tolist())
+        for b in range(B):
+            if cu[b + 1] == cu[b]:
+                continue
+            S = state[sl[b]].clone() if qs[b] > 0 else torch.zeros(C)
+            for t in range(cu[b], cu[b + 1]):
+                S = a[t] * S + g[t]
+                out[t] = S
+            state[sl[b]] = S
+        return (out * _act("gelu_tanh", yf)).to(x.dtype)
+    a = torch.empty(T, C, dtype=torch.float32, device=x.device)
+    g = torch.empty_like(a)
+    rc = _L().afm_rglru_gates(
+        _lib.ptr(a), _lib.ptr(g), _lib.ptr(u), _lib.ptr(wr), _lib.ptr(br),
+        _lib.ptr(wi), _lib.ptr(bi), _lib.ptr(rate), T, C, blocks, _code(u),
+        _lib.cur_stream())
+    _lib.check(rc, "afm_rglru_gates")
+    out = torch.empty(T, C, dtype=x.dtype, device=x.device)
+    lens = getattr(md, "seq_lens", None)
+    rc = _L().afm_rglru_scan(
+        _lib.ptr(out), _lib.ptr(state), _lib.ptr(a), _lib.ptr(g), _lib.ptr(y),
+        _rowstride(y), _lib.ptr(y_bias), _lib.ptr(md.cu_seqlens),
+        _lib.ptr(md.q_start), _lib.ptr(md.state_slots), B, C,
+        max(lens) if lens is not None else 1, _code(x), _lib.cur_stream())
+    _lib.check(rc, "afm_rglru_scan")
     return out
