@@ -12,6 +12,7 @@ from __future__ import annotations
 import os
 import subprocess
 import sys
+from concurrent.futures import ThreadPoolExecutor
 from pathlib import Path
 
 PKG_DIR = Path(__file__).resolve().parent
@@ -115,7 +116,7 @@ def _build_lib(lib: Path, sources, force: bool, verbose: bool) -> Path:
     import tempfile
     objdir = CSRC / ".obj"
     objdir.mkdir(exist_ok=True)
-    objs = []
+    objs, cmds = [], []
     for src in sources:
         sp = CSRC / src
         op = objdir / (src + ".o")
@@ -125,11 +126,13 @@ def _build_lib(lib: Path, sources, force: bool, verbose: bool) -> Path:
                 and all(op.stat().st_mtime > (CSRC / h).stat().st_mtime
                         for h in HEADERS)):
             continue
-        cmd = [
+        cmds.append([
             HIPCC, f"--offload-arch={ARCH}", *HIP_FLAGS,
             "-c", str(sp), "-o", str(op),
-        ]
-        _run(cmd, verbose)
+        ])
+    # the sources of a library compile side by side
+    with ThreadPoolExecutor(max_workers=min(4, max(1, len(cmds)))) as pool:
+        list(pool.map(lambda c: _run(c, verbose), cmds))
     # link to a temporary name and rename: a concurrent process never maps a
     # half-written library
     fd, tmp = tempfile.mkstemp(dir=str(lib.parent), prefix=lib.name + ".")
