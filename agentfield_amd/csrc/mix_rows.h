@@ -73,7 +73,7 @@ __device__ __forceinline__ void st2(S* p, float a, float b) {
 template <typename S> __device__ __forceinline__ float gelu_tanh(float a) {
   const float t = 0.7978845608028654f * (a + 0.044715f * a * a * a);
   if constexpr (sizeof(S) == 2)
-    return a - a * __frcp_rn(1.0f + __expf(2.0f * t));
+    return a - a * __builtin_amdgcn_rcpf(1.0f + __expf(2.0f * t));
   else
     return 0.5f * a * (1.0f + tanhf(t));
 }

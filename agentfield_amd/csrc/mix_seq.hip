@@ -249,7 +249,11 @@ __device__ __forceinline__ void load_slice(const S* row, int e0, int n,
   }
 }
 
-template <typename S, int GQ, bool VEC>
+// NK = 2 (differential attention, ex.vshare == 2): the workgroup's heads are
+// both maps of one value head, the first half on key head 2 gv, the second on
+// 2 gv + 1, so that a value row is read once for both; grid.y and G count
+// value heads, H all query heads.
+template <typename S, int GQ, bool VEC, int NK = 1>
 __global__ void __launch_bounds__(256) attn_rows_kernel(
     S* __restrict__ out, const S* __restrict__ q, const S* __restrict__ kc,
     const S* __restrict__ vc, const i32* __restrict__ bt,
@@ -274,7 +278,7 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(
   const int dkp = (dk + EPL - 1) / EPL * EPL;
   float* qs = r2s + 8;                         // [GQ][dkp] scaled queries
   const int t = blockIdx.x, g = blockIdx.y;
-  const int GV = G / ex.vshare, gv = g / ex.vshare;
+  const int GV = NK == 2 ? G : G / ex.vshare, gv = NK == 2 ? g : g / ex.vshare;
   const int hpg = H / G;
   const int zh = blockIdx.z / nsplit, sp = blockIdx.z % nsplit;
   const int h0 = g * hpg + zh * GQ;
@@ -327,7 +331,8 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(
     for (int kidx = threadIdx.x; kidx < nk; kidx += 256) {
       const int jv = tile0 + kidx;
       const int j = jv < wlo ? jv - vsh : jv;
-      const S* kr = kc + (((size_t)btr[j / page] * G + g) * page + (j % page)) * dk;
+      const S* kr = kc + (((size_t)btr[j / page] * G + g) * NK * page + (j % page)) * dk;
+      const S* kr1 = kr + (size_t)(NK - 1) * page * dk;    // the second map's
       float sco[GQ];
 #pragma unroll
       for (int gg = 0; gg < GQ; ++gg) sco[gg] = 0.f;
@@ -336,9 +341,16 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(
         float kv[EPL];
         load_slice<S, VEC>(kr, e0, dk, kv);
 #pragma unroll
-        for (int gg = 0; gg < GQ; ++gg)
+        for (int gg = 0; gg < GQ / NK; ++gg)
 #pragma unroll
           for (int e = 0; e < EPL; ++e) sco[gg] += qs[gg * dkp + e0 + e] * kv[e];
+        if constexpr (NK == 2) {
+          load_slice<S, VEC>(kr1, e0, dk, kv);
+#pragma unroll
+          for (int gg = GQ / 2; gg < GQ; ++gg)
+#pragma unroll
+            for (int e = 0; e < EPL; ++e) sco[gg] += qs[gg * dkp + e0 + e] * kv[e];
+        }
       }
 #pragma unroll
       for (int gg = 0; gg < GQ; ++gg)
@@ -750,6 +762,10 @@ static int launch_attention(void* out, const void* q, const void* kc,
   if (dk <= 64 * EPL && dv <= 64 * EPL) {
     auto clog2 = [](int n) { int l = 0; while ((1 << l) < n) ++l; return l; };
     const int lpk = clog2((dk + EPL - 1) / EPL), lpv = clog2((dv + EPL - 1) / EPL);
+    // both maps of a value head in one workgroup when its heads fit exactly
+    const int pq = ex.vshare == 2 ? H / G * 2 : 0;
+    const bool both = pq == 2 || pq == 4 || pq == 8;
+    if (both) G /= 2;
     const int hpg = H / G;
     const int gq = hpg >= 8 ? 8 : hpg > 2 ? 4 : hpg;   // 1, 2, 4 or 8
     const int dvp = EPL << lpv;
@@ -760,12 +776,20 @@ static int launch_attention(void* out, const void* q, const void* kc,
     const bool vec = dk % EPL == 0 && dv % EPL == 0 && ex.ldv % EPL == 0 &&
                      (uintptr_t)kc % 16 == 0 && (uintptr_t)vc % 16 == 0;
     dim3 grid(T, G, ((hpg + gq - 1) / gq) * nsplit);
-#define ROWS(GQ, VEC)                                                         \
-  attn_rows_kernel<S, GQ, VEC><<<grid, 256, sm, s>>>(                         \
+#define ROWS(GQ, ...)                                                         \
+  attn_rows_kernel<S, GQ, __VA_ARGS__><<<grid, 256, sm, s>>>(                 \
       (S*)out, (const S*)q, (const S*)kc, (const S*)vc, (const i32*)bt,       \
       (const i32*)row_seq, (const i32*)positions, scale, H, G, dk, dv, page,  \
       maxp, chunk, window, ldq, lpk, lpv, kt, nsplit, part_o, part_ml, ex)
-    if (vec) {
+    if (both) {
+      if (vec) {
+        if (gq == 2) ROWS(2, true, 2); else if (gq == 4) ROWS(4, true, 2);
+        else ROWS(8, true, 2);
+      } else {
+        if (gq == 2) ROWS(2, false, 2); else if (gq == 4) ROWS(4, false, 2);
+        else ROWS(8, false, 2);
+      }
+    } else if (vec) {
       if (gq == 1) ROWS(1, true); else if (gq == 2) ROWS(2, true);
       else if (gq == 4) ROWS(4, true); else ROWS(8, true);
     } else {

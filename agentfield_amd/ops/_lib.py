@@ -201,8 +201,8 @@ def _mix_sigs() -> dict:
                                   p],
         },
         "rglru": {
-            "afm_rglru_gates": [p, p, p, p, p, p, p, p, i, i, i, i, p],
-            "afm_rglru_scan": [p, p, p, p, p, i64, p, p, p, p, i, i, i, i, p],
+            "afm_rglru_gates": [p, p, p, p, p, p, p, i, i, i, i, p],
+            "afm_rglru_scan": [p, p, p, p, i64, p, p, p, p, i, i, i, i, p],
             "afm_rglru_step": [p, p, p, p, i64, p, p, p, p, i64, p, p, p, p,
                                p, p, p, p, i, i, i, i, p],
         },

@@ -415,7 +415,8 @@ def diff_attention(q: torch.Tensor, kcache: torch.Tensor,
         wgs = T * G2 * -(-hpg // 16)
         nsplit = max(1, min(16, 2048 // max(1, wgs), -(-reach // 64)))
     else:
-        wgs = T * G2 * -(-hpg // min(8, hpg))
+        # heads of both maps share a workgroup where they fit one exactly
+        wgs = T * G if hpg in (1, 2, 4) else T * G2 * -(-hpg // min(8, hpg))
         nsplit = max(1, min(8, 2048 // max(1, wgs), reach // 128))
         if max(dk, dv) > 64 * (16 // q.element_size()):
             nsplit = 1          # the kernel for such wide heads has no splits
@@ -1659,17 +1660,16 @@ def rglru(x: torch.Tensor, x_bias: torch.Tensor | None, y: torch.Tensor,
                 out[t] = S
             state[sl[b]] = S
         return (out * _act("gelu_tanh", yf)).to(x.dtype)
-    a = torch.empty(T, C, dtype=torch.float32, device=x.device)
-    g = torch.empty_like(a)
+    ag = torch.empty(T, C, 2, dtype=torch.float32, device=x.device)
     rc = _L().afm_rglru_gates(
-        _lib.ptr(a), _lib.ptr(g), _lib.ptr(u), _lib.ptr(wr), _lib.ptr(br),
-        _lib.ptr(wi), _lib.ptr(bi), _lib.ptr(rate), T, C, blocks, _code(u),
+        _lib.ptr(ag), _lib.ptr(u), _lib.ptr(wr), _lib.ptr(br), _lib.ptr(wi),
+        _lib.ptr(bi), _lib.ptr(rate), T, C, blocks, _code(u),
         _lib.cur_stream())
     _lib.check(rc, "afm_rglru_gates")
     out = torch.empty(T, C, dtype=x.dtype, device=x.device)
     lens = getattr(md, "seq_lens", None)
     rc = _L().afm_rglru_scan(
-        _lib.ptr(out), _lib.ptr(state), _lib.ptr(a), _lib.ptr(g), _lib.ptr(y),
+        _lib.ptr(out), _lib.ptr(state), _lib.ptr(ag), _lib.ptr(y),
         _rowstride(y), _lib.ptr(y_bias), _lib.ptr(md.cu_seqlens),
         _lib.ptr(md.q_start), _lib.ptr(md.state_slots), B, C,
         max(lens) if lens is not None else 1, _code(x), _lib.cur_stream())
