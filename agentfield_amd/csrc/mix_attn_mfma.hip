@@ -117,20 +117,25 @@ struct DiffTail {
   float lam, diff, eps;
 };
 
-template <int DKC, int DVT, bool VEC, int NH, int KT, bool DIFF = false>
+// LITE: no chunk, soft cap, distance bias or kept keys (window and sink
+// stay): what those terms keep alive costs the wide instances registers.
+template <int DKC, int DVT, bool VEC, int NH, int KT, bool DIFF = false,
+          bool LITE = false>
 __device__ __forceinline__ void attn_prefill_mfma_body(
     u16* __restrict__ out, const u16* __restrict__ q,
     const u16* __restrict__ kc, const u16* __restrict__ vc,
     const i32* __restrict__ bt, const i32* __restrict__ cu,
     const i32* __restrict__ q_start, const i32* __restrict__ tile_seq,
     const i32* __restrict__ tile_q0, float scale, int H, int G, int dk, int dv,
-    int page, int maxp, int chunk, int window, i64 ldq, const AttnExtra& ex,
+    int page, int maxp, int chunk_in, int window, i64 ldq, const AttnExtra& ex,
     const DiffTail& df = DiffTail{}) {
   constexpr int KS = DKC * 32 + 8;   // K row stride in LDS (elements)
   constexpr int VS = KT + 8;         // V^T / P row stride (KT tokens + pad)
   constexpr int NST = KT / 16;       // 16-key sub-tiles
   constexpr int NHF = KT / 32;       // 32-key halves of P V
   constexpr int NK = DIFF ? 2 : 1;
+  const int chunk = LITE ? 0 : chunk_in, first = LITE ? 0 : ex.first;
+  const bool biased = !LITE && ex.r1, capped = !LITE && ex.cap > 0.f;
   constexpr int XS = DVT * 16 + 4;   // row stride of the maps' exchange (floats)
   constexpr size_t KVB = sizeof(u16) * (NK * KT * KS + DVT * 16 * VS);
   constexpr size_t XB = DIFF ? sizeof(float) * 64 * XS : 0;
@@ -139,7 +144,7 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
   u16* k_lds = reinterpret_cast<u16*>(kv_lds);
   u16* v_lds = k_lds + NK * KT * KS;
   __shared__ u16 p_lds[NH * 4 * 16 * VS];
-  __shared__ float bias_lds[NH * 128];  // distance bias of this tile's distances
+  __shared__ float bias_lds[LITE ? 1 : NH * 128];  // distance bias of this tile's distances
   // page rows of every key of the tile
   __shared__ i32 row_lds[KT], vrow_lds[KT];
 
@@ -191,12 +196,12 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
 #pragma unroll
   for (int dt = 0; dt < DVT; ++dt) o_acc[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   u16* pw = p_lds + (hsel * 4 + wid) * 16 * VS;
-  const float r1 = ex.r1 ? ex.r1[h] : 0.f, r2 = ex.r1 ? ex.r2[h] : 0.f;
-  const float inv_cap = ex.cap > 0.f ? 1.0f / ex.cap : 0.f;
+  const float r1 = biased ? ex.r1[h] : 0.f, r2 = biased ? ex.r2[h] : 0.f;
+  const float inv_cap = capped ? 1.0f / ex.cap : 0.f;
 
   // always-visible leading keys that lie in front of the window are walked
   // first, in whole tiles from key 0; the window's tiles follow from b0
-  const int nfirst = (ex.first > 0 && lo > 0) ? min(ex.first, lo) : 0;
+  const int nfirst = (first > 0 && lo > 0) ? min(first, lo) : 0;
   const int a_end = (nfirst + KT - 1) / KT * KT;
   const int b0 = max(lo, a_end);
   for (int kv0 = nfirst > 0 ? 0 : lo; kv0 <= p_last;
@@ -207,7 +212,7 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
         gv, page, dk, dv, ex.ldv);
     // distance bias for every distance between a row and a key of the tile:
     // entry i is distance i + (p0 - kv0 - (KT-1)); keys ahead of a row are masked
-    if (ex.r1 && (threadIdx.x & 255) < 63 + KT) {     // each head its own table
+    if (biased && (threadIdx.x & 255) < 63 + KT) {     // each head its own table
       const int dist = (int)(threadIdx.x & 255) + p0 - kv0 - (KT - 1);
       bias_lds[hsel * 128 + (threadIdx.x & 255)] =
           dist > 0 ? attn_dist_bias(r1, r2, dist) : 0.f;
@@ -215,7 +220,7 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
     __syncthreads();
     // keys of this tile that any row of the wave may see
     if (!wave_live || kv0 > wp_last) continue;
-    if (window > 0 && kv0 + KT - 1 <= wp0 - window && kv0 >= ex.first) continue;
+    if (window > 0 && kv0 + KT - 1 <= wp0 - window && kv0 >= first) continue;
 
     // ---- S = Q K^T: 16-key sub-tiles ----
     f32x4 s_acc[NST];
@@ -244,9 +249,9 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
       for (int st = 0; st < NST; ++st) {
         const int j = kv0 + st * 16 + (lane & 15);
         float sv = s_acc[st][r] * scale;
-        if (ex.cap > 0.f) sv = attn_softcap_fast(sv, inv_cap, ex.cap);
-        if (ex.r1) sv -= bias_lds[hsel * 128 + (p - p0) - (j - kv0) + KT - 1];
-        sr[st] = (j <= p && (j >= rlo || j < ex.first)) ? sv : AF_NEG_INF;
+        if (capped) sv = attn_softcap_fast(sv, inv_cap, ex.cap);
+        if (biased) sv -= bias_lds[hsel * 128 + (p - p0) - (j - kv0) + KT - 1];
+        sr[st] = (j <= p && (j >= rlo || j < first)) ? sv : AF_NEG_INF;
         tmax = fmaxf(tmax, sr[st]);
       }
       tmax = group16_max_f32(tmax);
@@ -357,23 +362,24 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
     out, q, kc, vc, bt, cu, q_start, tile_seq, tile_q0, scale, H, G, dk, dv,   \
     page, maxp, chunk, window, ldq, ex
 
-template <int DKC, int DVT, bool VEC, int NH, int KT = 64>
+template <int DKC, int DVT, bool VEC, int NH, int KT = 64, bool LITE = false>
 __global__ void __launch_bounds__(256 * NH) attn_prefill_mfma_kernel(AF_APM_PARAMS) {
-  attn_prefill_mfma_body<DKC, DVT, VEC, NH, KT>(AF_APM_ARGS);
+  attn_prefill_mfma_body<DKC, DVT, VEC, NH, KT, false, LITE>(AF_APM_ARGS);
 }
 
 // The widest instance keeps 16 x 512 output accumulators and an 18-fragment
 // query per wave: two waves per SIMD (the eight waves of one workgroup) is all
 // a CU can hold of it, so it may use their full register share.
+template <bool LITE>
 __global__ void __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(2, 2)))
 attn_prefill_mfma_wide_pair_kernel(AF_APM_PARAMS) {
-  attn_prefill_mfma_body<18, 32, true, 2, 32>(AF_APM_ARGS);
+  attn_prefill_mfma_body<18, 32, true, 2, 32, false, LITE>(AF_APM_ARGS);
 }
 
 template <int DKC, int DVT, bool VEC, int KT = 64>
 __global__ void __launch_bounds__(512) diff_prefill_mfma_kernel(AF_APM_PARAMS,
                                                                 DiffTail df) {
-  attn_prefill_mfma_body<DKC, DVT, VEC, 2, KT, true>(AF_APM_ARGS, df);
+  attn_prefill_mfma_body<DKC, DVT, VEC, 2, KT, true, true>(AF_APM_ARGS, df);
 }
 
 // ------------------------------------------------ single rows, many heads
@@ -624,6 +630,7 @@ AF_EXPORT int afm_attn_prefill_mfma(
                      cap, ldv, keep_first, vshare};
   // two heads per workgroup when a K/V group has an even number of them
   const bool pair = vec && (H / G) % 2 == 0;
+  const bool lite = chunk <= 0 && cap <= 0.f && !r1 && keep_first == 0;
   hipStream_t s = (hipStream_t)stream;
 #define APM(DKC, DVT, VEC, NH, ...)                                            \
   attn_prefill_mfma_kernel<DKC, DVT, VEC, NH, ##__VA_ARGS__>                   \
@@ -636,16 +643,19 @@ AF_EXPORT int afm_attn_prefill_mfma(
   // the widest heads pair up over 32-key tiles: two heads' 64-key tiles are
   // 164 KB of LDS
   if (dk > 320 || dv > 256) {
-    if (pair)
-      attn_prefill_mfma_wide_pair_kernel<<<dim3(ntiles, H / 2), 512, 0, s>>>(
-          (u16*)out, (const u16*)q, (const u16*)kc, (const u16*)vc,
-          (const i32*)bt, (const i32*)cu, (const i32*)q_start,
-          (const i32*)tile_seq, (const i32*)tile_q0, scale, H, G, dk, dv, page,
-          maxp, chunk, window, ldq, ex);
+#define APW(LITE)                                                              \
+  attn_prefill_mfma_wide_pair_kernel<LITE><<<dim3(ntiles, H / 2), 512, 0, s>>>(\
+      (u16*)out, (const u16*)q, (const u16*)kc, (const u16*)vc,                \
+      (const i32*)bt, (const i32*)cu, (const i32*)q_start,                     \
+      (const i32*)tile_seq, (const i32*)tile_q0, scale, H, G, dk, dv, page,    \
+      maxp, chunk, window, ldq, ex)
+    if (pair && lite) APW(true);
+    else if (pair) APW(false);
+#undef APW
     else
       APM(18, 32, true, 1);
   }
-  else if (dk > 128 || dv > 128) { if (pair) APM(10, 16, true, 2); else APM(10, 16, true, 1); }
+  else if (dk > 128 || dv > 128) { if (pair && lite) APM(10, 16, true, 2, 64, true); else if (pair) APM(10, 16, true, 2); else APM(10, 16, true, 1); }
   else if (small && pair) APM(2, 4, true, 2);
   else if (small && vec) APM(2, 4, true, 1);
   else if (small) APM(2, 4, false, 1);
