@@ -214,14 +214,16 @@ def qk_norm_cache(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
 
 def _row_tiles(lens, rows: int, device):
     """Tile map of packed chunks for the tile kernels: (tiles, sequence of
-    every tile, its first row inside the chunk)."""
-    ts, tq = [], []
-    for b, ln in enumerate(lens):
-        for q0 in range(0, ln, rows):
-            ts.append(b)
-            tq.append(q0)
-    return (len(ts), torch.tensor(ts, dtype=torch.int32, device=device),
-            torch.tensor(tq, dtype=torch.int32, device=device))
+    every tile, its first row inside the chunk).  Late rows see the most keys
+    and go first, so that a launch ends on short tiles; sequences alternate,
+    which spreads them over the XCDs and keeps each one's keys in few L2s."""
+    tiles = sorted((-q0, b) for b, ln in enumerate(lens)
+                   for q0 in range(0, ln, rows))
+    return (len(tiles),
+            torch.tensor([b for _q, b in tiles], dtype=torch.int32,
+                         device=device),
+            torch.tensor([-q for q, _b in tiles], dtype=torch.int32,
+                         device=device))
 
 
 def masked_attention(q: torch.Tensor, kcache: torch.Tensor,
