@@ -17,6 +17,10 @@
 // vshare > 1: the value pages have G / vshare heads, each serving vshare
 // neighbouring key heads (differential attention: the two maps of a K/V head
 // have keys of their own over the same values).
+//
+// gate: one output-gate logit per (row, head) in the storage dtype, row stride
+// ldg; a head's output is multiplied by the logit's sigmoid.  ldo is the row
+// stride of the output in elements (at least H * dv).
 #pragma once
 #include "common.h"
 
@@ -28,7 +32,18 @@ struct AttnExtra {
   i64 ldv;
   int first;           // 0: no always-visible leading keys
   int vshare;          // key heads per value head
+  const void* gate;    // [T, H] at stride ldg, or null
+  i64 ldg, ldo;
 };
+
+template <typename S>
+__device__ __forceinline__ float attn_head_gate(const AttnExtra& ex, size_t t, int h) {
+  if (!ex.gate) return 1.0f;
+  float z;
+  if constexpr (sizeof(S) == 2) z = bf2f(static_cast<const u16*>(ex.gate)[t * ex.ldg + h]);
+  else z = static_cast<const float*>(ex.gate)[t * ex.ldg + h];
+  return 1.0f / (1.0f + expf(-z));
+}
 
 // exact forms (fp32 storage and the row kernels)
 __device__ __forceinline__ float attn_softcap(float s, float cap) {

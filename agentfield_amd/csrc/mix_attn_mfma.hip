@@ -341,8 +341,8 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
   for (int r = 0; r < 4; ++r) {
     const int row = q0 + wrow0 + (lane >> 4) * 4 + r;
     if (row >= len) continue;
-    const float inv = l[r] > 0.f ? 1.0f / l[r] : 0.f;
-    u16* op = out + ((size_t)(r0 + row) * H + h) * dv;
+    const float inv = (l[r] > 0.f ? 1.0f / l[r] : 0.f) * attn_head_gate<u16>(ex, r0 + row, h);
+    u16* op = out + (size_t)(r0 + row) * ex.ldo + (size_t)h * dv;
 #pragma unroll
     for (int dt = 0; dt < DVT; ++dt) {
       const int d = dt * 16 + (lane & 15);
@@ -583,11 +583,13 @@ __global__ void __launch_bounds__(256) attn_heads_mfma_kernel(
     if (hr >= nrows) continue;
     const size_t th = (size_t)t * H + hbase + hr;
     if (!part_o) {
-      const float inv = l[r] > 0.f ? 1.0f / l[r] : 0.f;
+      const int head = hbase + hr;
+      const float inv = (l[r] > 0.f ? 1.0f / l[r] : 0.f) * attn_head_gate<u16>(ex, t, head);
+      u16* op = out + (size_t)t * ex.ldo + (size_t)head * dv;
 #pragma unroll
       for (int dw = 0; dw < DVW; ++dw) {
         const int d = (wid * DVW + dw) * 16 + (lane & 15);
-        if (d < dv) out[th * dv + d] = f2bf(o_acc[dw][r] * inv);
+        if (d < dv) op[d] = f2bf(o_acc[dw][r] * inv);
       }
     } else {
 #pragma unroll
@@ -607,15 +609,16 @@ __global__ void __launch_bounds__(256) attn_heads_mfma_kernel(
 
 // q [T, H*dk] bf16 rows at stride ldq; caches [P, G, page, dk|dv] bf16;
 // tile map (tile_seq, tile_q0): workgroup i covers chunk rows
-// [q0, q0 + 64) of sequence tile_seq[i].  out [T, H*dv] bf16.
+// [q0, q0 + 64) of sequence tile_seq[i].  out [T, H*dv] bf16 at row stride ldo.
 AF_EXPORT int afm_attn_prefill_mfma(
     void* out, const void* q, const void* kc, const void* vc, const void* bt,
     const void* cu, const void* q_start, const void* tile_seq,
     const void* tile_q0, float scale, int ntiles, int H, int G, int dk, int dv,
     int page, int maxp, int chunk, int window, i64 ldq, const void* sink,
     float cap, const void* r1, const void* r2, i64 ldv, int keep_first,
-    int vshare, void* stream) {
+    int vshare, const void* gate, i64 ldg, i64 ldo, void* stream) {
   if (ntiles == 0) return 0;
+  if (ldo < (i64)H * dv || (gate && ldg < H)) return 9003;
   if (keep_first < 0 || vshare < 1 || G % vshare) return 9003;
   if (G <= 0 || H % G || dk < 1 || dv < 1) return 9003;
   if (ldv < dv || cap < 0.f || ((r1 == nullptr) != (r2 == nullptr))) return 9003;
@@ -627,7 +630,7 @@ AF_EXPORT int afm_attn_prefill_mfma(
   // to the row kernel
   if (dk > 576 || dv > 512 || ((dk > 128 || dv > 128) && !vec)) return 9004;
   const AttnExtra ex{(const float*)sink, (const float*)r1, (const float*)r2,
-                     cap, ldv, keep_first, vshare};
+                     cap, ldv, keep_first, vshare, gate, ldg, ldo};
   // two heads per workgroup when a K/V group has an even number of them
   const bool pair = vec && (H / G) % 2 == 0;
   const bool lite = chunk <= 0 && cap <= 0.f && !r1 && keep_first == 0;
@@ -707,8 +710,9 @@ AF_EXPORT int afm_attn_heads_mfma(
     int G, int dk, int dv, int page, int maxp, int chunk, int window, i64 ldq,
     int nsplit, void* part_o, void* part_ml, const void* sink, float cap,
     const void* r1, const void* r2, i64 ldv, int keep_first, int vshare,
-    void* stream) {
+    const void* gate, i64 ldg, i64 ldo, void* stream) {
   if (T == 0) return 0;
+  if (out && (ldo < (i64)H * dv || (gate && ldg < H))) return 9003;
   if (keep_first < 0 || vshare < 1 || G % vshare) return 9003;
   if (G <= 0 || H % G || dk < 1 || dv < 1) return 9003;
   if (ldv < dv || cap < 0.f || ((r1 == nullptr) != (r2 == nullptr))) return 9003;
@@ -719,7 +723,7 @@ AF_EXPORT int afm_attn_heads_mfma(
                    ((uintptr_t)vc % 16 == 0);
   if (dk > 576 || dv > 512 || ((dk > 128 || dv > 128) && !vec)) return 9004;
   const AttnExtra ex{(const float*)sink, (const float*)r1, (const float*)r2,
-                     cap, ldv, keep_first, vshare};
+                     cap, ldv, keep_first, vshare, gate, ldg, ldo};
   const int hpg = H / G;
   dim3 grid(T, G * ((hpg + 15) / 16), nsplit), blk(256);
   hipStream_t s = (hipStream_t)stream;

@@ -131,6 +131,26 @@ __global__ void __launch_bounds__(256) conv_state_kernel(
 
 }  // namespace
 
+// The slots' move to the last taps-1 inputs alone (for convolutions that other
+// kernels evaluate).
+AF_EXPORT int afm_conv_state(void* state, const void* in, i64 ldi,
+                             const void* cu, const void* q_start,
+                             const void* sslot, int B, int C, int taps, int dt,
+                             void* stream) {
+  if (B == 0 || taps <= 1) return 0;
+  if (!state) return 9003;
+  hipStream_t s = (hipStream_t)stream;
+#define CS(ST)                                                               \
+  conv_state_kernel<ST><<<grid_for((i64)B * C), 256, 0, s>>>((ST*)state,     \
+      (const ST*)in, ldi, (const i32*)cu, (const i32*)q_start,               \
+      (const i32*)sslot, B, C, taps)
+  if (dt == 0) CS(u16);
+  else if (dt == 1) CS(float);
+  else return 9002;
+#undef CS
+  return af_last_err();
+}
+
 AF_EXPORT int afm_causal_conv(void* out, const void* in, i64 ldi,
                               const void* w, const void* bias,
                               const void* in_bias, void* state,

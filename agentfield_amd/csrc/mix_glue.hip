@@ -82,6 +82,51 @@ __global__ void __launch_bounds__(256) embed_kernel(
     dst[i] = ldf<S>(src + i) * scale + (add ? add[i] : 0.f);
 }
 
+// x = table[token] + pairs[row of (previous token, token)]: the pair row is
+// (previous * mul_prev + token * mul_cur) mod buckets, row `buckets` where a
+// sequence starts.  The token before a chunk comes from the sequence's slot of
+// `prev` [slots].  STEP: every chunk is a single row, which leaves its token
+// in the slot itself; longer chunks leave it through last_token_kernel.
+template <typename S, int V, bool STEP>
+__global__ void __launch_bounds__(256) embed_pairs_kernel(
+    float* __restrict__ out, const S* __restrict__ table,
+    const S* __restrict__ pairs, const i32* __restrict__ ids, i32* prev,
+    const i32* __restrict__ row_seq, const i32* __restrict__ cu,
+    const i32* __restrict__ q_start, const i32* __restrict__ sslot,
+    i64 mul_prev, i64 mul_cur, i64 buckets, int W) {
+  const int t = blockIdx.x;
+  const int b = row_seq[t];
+  const int k = t - cu[b];
+  const i64 tok = ids[t];
+  i64 row = buckets;
+  if (k > 0 || q_start[b] > 0) {
+    const i64 before = k > 0 ? ids[t - 1] : prev[sslot[b]];
+    row = (before * mul_prev + tok * mul_cur) % buckets;
+    if (row < 0) row += buckets;
+  }
+  if (STEP) {
+    __syncthreads();                       // every thread has read the slot
+    if (threadIdx.x == 0) prev[sslot[b]] = (i32)tok;
+  }
+  const S* a = table + (size_t)tok * W;
+  const S* p = pairs + (size_t)row * W;
+  for (int i = threadIdx.x * V; i < W; i += 256 * V) {
+    float av[4], pv[4];
+    ldv<S, V>(a + i, av);
+    ldv<S, V>(p + i, pv);
+#pragma unroll
+    for (int j = 0; j < V; ++j) av[j] += pv[j];
+    stv<float, V>(out + (size_t)t * W + i, av);
+  }
+}
+
+__global__ void __launch_bounds__(256) last_token_kernel(
+    i32* __restrict__ prev, const i32* __restrict__ ids,
+    const i32* __restrict__ cu, const i32* __restrict__ sslot, int B) {
+  const int b = blockIdx.x * 256 + threadIdx.x;
+  if (b < B && cu[b + 1] > cu[b]) prev[sslot[b]] = ids[cu[b + 1] - 1];
+}
+
 __global__ void __launch_bounds__(256) add_rows_kernel(
     float* __restrict__ x, const float* __restrict__ other,
     const float* __restrict__ vec, i64 n, int W) {
@@ -384,6 +429,129 @@ __global__ void __launch_bounds__(256) xielu_kernel(
   }
 }
 
+// Residual add of a layer whose sublayers share one input, and the RMSNorm in
+// front of the next layer, in one pass over the row:
+//   u = a + sum_r wts[r] ys[pos[r]] + (sum_i idw[i]) hin
+//   x += mult * u (+ vec);   h = x / sqrt(mean(x^2) + eps) * w
+// a: what sits in token order (or null); ys: rows in another order, pos < 0
+// skipped (top 0: none); hin: the layer's own input under the weights idw [nid]
+// at row stride ldi (nid 0: none); vec: one fp32 row; h null: no norm.
+// REG: the row fits 4 passes of the workgroup and waits in registers for the
+// sum; otherwise it is read again.
+template <typename S, int V, int NT, bool REG>
+__global__ void __launch_bounds__(NT) residual_norm_kernel(
+    float* __restrict__ x, S* __restrict__ h, const S* __restrict__ a, i64 lda,
+    const S* __restrict__ ys, const i32* __restrict__ pos,
+    const float* __restrict__ wts, int top, const S* __restrict__ hin,
+    const float* __restrict__ idw, i64 ldi, int nid, float mult,
+    const float* __restrict__ vec, const S* __restrict__ w, float eps, int W) {
+  __shared__ float red[NT / 64];
+  const int t = blockIdx.x;
+  float* xr = x + (size_t)t * W;
+  float fid = 0.f;
+  for (int i = 0; i < nid; ++i) fid += idw[(size_t)t * ldi + i];
+  const i32* pr = pos + (size_t)t * top;
+  const float* wr = wts + (size_t)t * top;
+  auto update = [&](int i, float (&xv)[4]) {
+    float u[4] = {0.f, 0.f, 0.f, 0.f}, v[4];
+    ldv<float, V>(xr + i, xv);
+    if (a) ldv<S, V>(a + (size_t)t * lda + i, u);
+    for (int r = 0; r < top; ++r) {
+      const int p = pr[r];
+      if (p < 0) continue;
+      const float f = wr[r];
+      ldv<S, V>(ys + (size_t)p * W + i, v);
+#pragma unroll
+      for (int j = 0; j < V; ++j) u[j] += f * v[j];
+    }
+    if (fid != 0.f) {
+      ldv<S, V>(hin + (size_t)t * W + i, v);
+#pragma unroll
+      for (int j = 0; j < V; ++j) u[j] += fid * v[j];
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) xv[j] += mult * u[j];
+    if (vec) {
+      ldv<float, V>(vec + i, v);
+#pragma unroll
+      for (int j = 0; j < V; ++j) xv[j] += v[j];
+    }
+    stv<float, V>(xr + i, xv);
+  };
+  float xs[SWN_IT][4];
+  float ss = 0.f;
+  if constexpr (REG) {
+#pragma unroll
+    for (int p = 0; p < SWN_IT; ++p) {
+      const int i = (p * NT + threadIdx.x) * V;
+      if (i < W) {
+        update(i, xs[p]);
+#pragma unroll
+        for (int j = 0; j < V; ++j) ss += xs[p][j] * xs[p][j];
+      }
+    }
+  } else {
+    for (int i = threadIdx.x * V; i < W; i += NT * V) {
+      update(i, xs[0]);
+#pragma unroll
+      for (int j = 0; j < V; ++j) ss += xs[0][j] * xs[0][j];
+    }
+  }
+  if (!h) return;
+  ss = wave_sum_f32(ss);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
+  __syncthreads();
+  ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NT / 64; ++i) ss += red[i];
+  const float rs = 1.0f / sqrtf(ss / (float)W + eps);
+  float wv[4];
+  if constexpr (REG) {
+#pragma unroll
+    for (int p = 0; p < SWN_IT; ++p) {
+      const int i = (p * NT + threadIdx.x) * V;
+      if (i < W) {
+        ldv<S, V>(w + i, wv);
+#pragma unroll
+        for (int j = 0; j < V; ++j) wv[j] *= xs[p][j] * rs;
+        stv<S, V>(h + (size_t)t * W + i, wv);
+      }
+    }
+  } else {
+    for (int i = threadIdx.x * V; i < W; i += NT * V) {
+      ldv<float, V>(xr + i, xs[0]);          // written by the same thread
+      ldv<S, V>(w + i, wv);
+#pragma unroll
+      for (int j = 0; j < V; ++j) wv[j] *= xs[0][j] * rs;
+      stv<S, V>(h + (size_t)t * W + i, wv);
+    }
+  }
+}
+
+// out = max(z, 0)^2 * f, rows of z at stride ldz, of out at ldo.  f is 1 in the
+// first `lead` columns, then rw[t, (c - lead) / unit] (rw null: 1 everywhere).
+template <typename S, int V>
+__global__ void __launch_bounds__(256) relu2_kernel(
+    S* __restrict__ out, i64 ldo, const S* __restrict__ z, i64 ldz,
+    const float* __restrict__ rw, i64 ldrw, int lead, int unit, int T, int F) {
+  const i64 per = F / V;
+  const i64 total = (i64)T * per;
+  for (i64 i = (i64)blockIdx.x * 256 + threadIdx.x; i < total;
+       i += (i64)gridDim.x * 256) {
+    const i64 t = i / per;
+    const int c = (int)(i % per) * V;
+    const float f = (rw && c >= lead) ? rw[t * ldrw + (c - lead) / unit] : 1.0f;
+    float v[4];
+    ldv<S, V>(z + t * ldz + c, v);
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      const float r = fmaxf(v[j], 0.f);
+      v[j] = r * r * f;
+    }
+    stv<S, V>(out + t * ldo + c, v);
+  }
+}
+
 // One wave per (row, head): RMS over dv of fp32 o, * weight, * silu(gate)
 // (SIG: * sigmoid(gate)).
 template <typename S, int V, bool SIG>
@@ -590,15 +758,16 @@ __global__ void __launch_bounds__(256) glu_kernel(
 // Sigmoid router with score correction and group-limited top-k, one wave per
 // token.  z [T, E] fp32 logits; s = sigmoid(z); choice = s + corr.  With
 // n_groups > 0 the experts form n_groups equal groups of neighbours, a
-// group's score is the sum of its two largest choice scores, and experts
-// outside the best `keep` groups cannot be chosen.  The `top` largest choice
+// group's score is the sum of its two largest choice scores (gtop 1: its
+// largest choice score), and experts outside the best `keep` groups cannot be chosen.  The `top` largest choice
 // scores win (ties: lower index); weights = s / (sum of chosen s + 1e-20) *
 // scale.  Outputs idx [T, top] i32, wts [T, top] fp32 and, optionally, the
 // dense form wd [T, E] fp32 (zero for experts not chosen).
 __global__ void __launch_bounds__(64) moe_route_kernel(
     i32* __restrict__ idx, float* __restrict__ wts, float* __restrict__ wd,
     const float* __restrict__ z, const float* __restrict__ corr, int E,
-    int top, int n_groups, int keep, float scale, int softmax, int renorm) {
+    int top, int n_groups, int keep, float scale, int softmax, int renorm,
+    int gtop) {
   extern __shared__ float sh[];
   float* sig = sh;             // [E]
   float* choice = sh + E;      // [E]
@@ -631,7 +800,7 @@ __global__ void __launch_bounds__(64) moe_route_kernel(
         if (c > a) { b = a; a = c; }
         else if (c > b) b = c;
       }
-      gsc[g] = size > 1 ? a + b : a;
+      gsc[g] = size > 1 && gtop > 1 ? a + b : a;
     }
     __syncthreads();
     for (int g = lane; g < n_groups; g += 64) {
@@ -675,20 +844,27 @@ __global__ void __launch_bounds__(64) moe_route_kernel(
   }
 }
 
-// y[t] = sum_r wts[t, r] * ys[pos[t*top + r]] (+ shared[t]) in fp32, the sum
-// taken in the order r = 0 .. top-1.  ys rows sit in expert-sorted order; pos
-// is the inverse of that sort.
+// y[t] = sum_r wts[t, r] * ys[pos[t*top + r]] (+ shared[t]) (+ (sum_i idw[t, i])
+// hin[t]) in fp32, the sum taken in the order r = 0 .. top-1.  ys rows sit in
+// expert-sorted order; pos is the inverse of that sort, negative for choices
+// without a row.  idw [nid] at row stride ldi: the weights of experts whose
+// output is their input hin.
 template <typename S>
 __global__ void __launch_bounds__(256) moe_combine_kernel(
     float* __restrict__ y, const S* __restrict__ ys,
     const i32* __restrict__ pos, const float* __restrict__ wts,
-    const S* __restrict__ shared, int top, int W) {
+    const S* __restrict__ shared, const S* __restrict__ hin,
+    const float* __restrict__ idw, i64 ldi, int nid, int top, int W) {
   const int t = blockIdx.x;
+  float fid = 0.f;
+  for (int i = 0; i < nid; ++i) fid += idw[(size_t)t * ldi + i];
   for (int i = threadIdx.x; i < W; i += 256) {
     float acc = shared ? ldf<S>(shared + (size_t)t * W + i) : 0.f;
-    for (int r = 0; r < top; ++r)
-      acc += wts[(size_t)t * top + r] *
-             ldf<S>(ys + (size_t)pos[(size_t)t * top + r] * W + i);
+    for (int r = 0; r < top; ++r) {
+      const int p = pos[(size_t)t * top + r];
+      if (p >= 0) acc += wts[(size_t)t * top + r] * ldf<S>(ys + (size_t)p * W + i);
+    }
+    if (fid != 0.f) acc += fid * ldf<S>(hin + (size_t)t * W + i);
     y[(size_t)t * W + i] = acc;
   }
 }
@@ -722,6 +898,36 @@ AF_EXPORT int afm_embed(void* out, const void* table, const void* ids,
           (const i32*)ids, (const float*)add, scale, W)),
       (embed_kernel<float><<<T, 256, 0, s>>>((float*)out, (const float*)table,
           (const i32*)ids, (const float*)add, scale, W)));
+  return af_last_err();
+}
+
+// prev [slots] i32; step: every chunk is one row.
+AF_EXPORT int afm_embed_pairs(void* out, const void* table, const void* pairs,
+                              const void* ids, void* prev, const void* row_seq,
+                              const void* cu, const void* q_start,
+                              const void* sslot, i64 mul_prev, i64 mul_cur,
+                              i64 buckets, int T, int B, int W, int step,
+                              int dt, void* stream) {
+  if (T == 0) return 0;
+  if (buckets < 1 || !prev) return 9003;
+  hipStream_t s = (hipStream_t)stream;
+  const bool vec = W % 4 == 0 && aligned16(out, table, pairs);
+#define EP(ST, V, SP)                                                         \
+  embed_pairs_kernel<ST, V, SP><<<T, 256, 0, s>>>((float*)out,                \
+      (const ST*)table, (const ST*)pairs, (const i32*)ids, (i32*)prev,        \
+      (const i32*)row_seq, (const i32*)cu, (const i32*)q_start,               \
+      (const i32*)sslot, mul_prev, mul_cur, buckets, W)
+#define EPV(ST)                                                               \
+  do {                                                                        \
+    if (vec) { if (step) EP(ST, 4, true); else EP(ST, 4, false); }            \
+    else { if (step) EP(ST, 1, true); else EP(ST, 1, false); }                \
+  } while (0)
+  MIX_DISPATCH(dt, EPV(u16), EPV(float));
+#undef EPV
+#undef EP
+  if (!step)
+    last_token_kernel<<<(B + 255) / 256, 256, 0, s>>>(
+        (i32*)prev, (const i32*)ids, (const i32*)cu, (const i32*)sslot, B);
   return af_last_err();
 }
 
@@ -917,6 +1123,69 @@ AF_EXPORT int afm_sandwich_norm(void* x, void* h, const void* y, i64 ldy,
   return af_last_err();
 }
 
+// x [T, W] fp32 in place; a at row stride lda, hin [T, W], ys rows of W in the
+// storage dtype; h (or null) [T, W] in the storage dtype.
+AF_EXPORT int afm_residual_norm(void* x, void* h, const void* a, i64 lda,
+                                const void* ys, const void* pos,
+                                const void* wts, int top, const void* hin,
+                                const void* idw, i64 ldi, int nid, float mult,
+                                const void* vec, const void* w, float eps,
+                                int T, int W, int dt, void* stream) {
+  if (T == 0) return 0;
+  if (h && !w) return 9003;
+  if (top < 0 || (top > 0 && (!ys || !pos || !wts))) return 9003;
+  if (nid < 0 || (nid > 0 && (!hin || !idw))) return 9003;
+  hipStream_t s = (hipStream_t)stream;
+  const bool vv = W % 4 == 0 && lda % 4 == 0 &&
+                  aligned16(x, h, a, ys, hin, vec, w);
+  const int cols = W / (vv ? 4 : 1);
+  // few rows of many columns: one column group per thread
+  const bool wide = T <= 512 && cols > 256;
+#define RNK(ST, V, NT, R)                                                    \
+  residual_norm_kernel<ST, V, NT, R><<<T, NT, 0, s>>>((float*)x, (ST*)h,     \
+      (const ST*)a, lda, (const ST*)ys, (const i32*)pos, (const float*)wts,  \
+      top, (const ST*)hin, (const float*)idw, ldi, nid, mult,                \
+      (const float*)vec, (const ST*)w, eps, W)
+#define RNR(ST, V)                                                           \
+  do {                                                                       \
+    if (wide && cols <= SWN_IT * 1024) RNK(ST, V, 1024, true);               \
+    else if (!wide && cols <= SWN_IT * 256) RNK(ST, V, 256, true);           \
+    else RNK(ST, V, 256, false);                                             \
+  } while (0)
+#define RN(ST)                                                               \
+  do { if (vv) RNR(ST, 4); else RNR(ST, 1); } while (0)
+  MIX_DISPATCH(dt, RN(u16), RN(float));
+#undef RN
+#undef RNR
+#undef RNK
+  return af_last_err();
+}
+
+// z, out [T, F] at row strides ldz, ldo; rw (or null) at row stride ldrw.
+AF_EXPORT int afm_relu2(void* out, i64 ldo, const void* z, i64 ldz,
+                        const void* rw, i64 ldrw, int lead, int unit, int T,
+                        int F, int dt, void* stream) {
+  if (T == 0 || F == 0) return 0;
+  if (lead < 0 || unit < 1 ||
+      (rw && F > lead && ((F - lead) % unit || ldrw < (F - lead) / unit)))
+    return 9003;
+  hipStream_t s = (hipStream_t)stream;
+  const bool vec = F % 4 == 0 && ldz % 4 == 0 && ldo % 4 == 0 &&
+                   (!rw || (lead % 4 == 0 && unit % 4 == 0)) &&
+                   (uintptr_t)out % (dt ? 16 : 8) == 0 &&
+                   (uintptr_t)z % (dt ? 16 : 8) == 0;
+  const i64 total = (i64)T * (vec ? F / 4 : F);
+  const int grid = (int)((total + 255) / 256 < 16384 ? (total + 255) / 256 : 16384);
+#define R2(S, V)                                                             \
+  relu2_kernel<S, V><<<grid, 256, 0, s>>>((S*)out, ldo, (const S*)z, ldz,    \
+      (const float*)rw, ldrw, lead, unit, T, F)
+  if (dt == 0) { if (vec) R2(u16, 4); else R2(u16, 1); }
+  else if (dt == 1) { if (vec) R2(float, 4); else R2(float, 1); }
+  else return 9002;
+#undef R2
+  return af_last_err();
+}
+
 AF_EXPORT int afm_xielu(void* out, const void* z, i64 ldz, const void* coef,
                         int T, int F, int dt, void* stream) {
   if (T == 0 || F == 0) return 0;
@@ -972,8 +1241,9 @@ AF_EXPORT int afm_glu(void* out, i64 ldo, i64 ldo_in, const void* g,
 AF_EXPORT int afm_moe_route(void* idx, void* wts, void* wd, const void* z,
                             const void* corr, int T, int E, int top,
                             int n_groups, int keep, float scale, int softmax,
-                            int renorm, void* stream) {
+                            int renorm, int gtop, void* stream) {
   if (T == 0) return 0;
+  if (gtop < 1 || gtop > 2) return 9003;
   if (E < 1 || top < 1 || top > E) return 9003;
   if (n_groups > 0 && (E % n_groups != 0 || keep < 1)) return 9003;
   const size_t sm = (size_t)(2 * E + (n_groups > 0 ? n_groups : 0)) *
@@ -981,19 +1251,25 @@ AF_EXPORT int afm_moe_route(void* idx, void* wts, void* wd, const void* z,
   if (sm > 60000) return 9004;
   moe_route_kernel<<<T, 64, sm, (hipStream_t)stream>>>(
       (i32*)idx, (float*)wts, (float*)wd, (const float*)z, (const float*)corr,
-      E, top, n_groups, keep, scale, softmax, renorm);
+      E, top, n_groups, keep, scale, softmax, renorm, gtop);
   return af_last_err();
 }
 
 AF_EXPORT int afm_moe_combine(void* y, const void* ys, const void* pos,
-                              const void* wts, const void* shared, int T,
-                              int top, int W, int dt, void* stream) {
+                              const void* wts, const void* shared,
+                              const void* hin, const void* idw, i64 ldi,
+                              int nid, int T, int top, int W, int dt,
+                              void* stream) {
   if (T == 0) return 0;
+  if (top < 0 || nid < 0 || (nid > 0 && (!hin || !idw))) return 9003;
+  if (top > 0 && (!ys || !pos || !wts)) return 9003;
   hipStream_t s = (hipStream_t)stream;
   MIX_DISPATCH(dt,
       (moe_combine_kernel<u16><<<T, 256, 0, s>>>((float*)y, (const u16*)ys,
-          (const i32*)pos, (const float*)wts, (const u16*)shared, top, W)),
+          (const i32*)pos, (const float*)wts, (const u16*)shared,
+          (const u16*)hin, (const float*)idw, ldi, nid, top, W)),
       (moe_combine_kernel<float><<<T, 256, 0, s>>>((float*)y, (const float*)ys,
-          (const i32*)pos, (const float*)wts, (const float*)shared, top, W)));
+          (const i32*)pos, (const float*)wts, (const float*)shared,
+          (const float*)hin, (const float*)idw, ldi, nid, top, W)));
   return af_last_err();
 }

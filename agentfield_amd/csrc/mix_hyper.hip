@@ -296,27 +296,6 @@ __global__ void __launch_bounds__(256) canon_state_kernel(
   }
 }
 
-// out = max(z, 0)^2, rows of z at stride ldz.
-template <typename S, int V>
-__global__ void __launch_bounds__(256) relu2_kernel(
-    S* __restrict__ out, const S* __restrict__ z, i64 ldz, int T, int F) {
-  const i64 per = F / V;
-  const i64 total = (i64)T * per;
-  for (i64 i = (i64)blockIdx.x * 256 + threadIdx.x; i < total;
-       i += (i64)gridDim.x * 256) {
-    const i64 t = i / per;
-    const int c = (int)(i % per) * V;
-    float v[4];
-    ldv<S, V>(z + t * ldz + c, v);
-#pragma unroll
-    for (int j = 0; j < V; ++j) {
-      const float r = fmaxf(v[j], 0.f);
-      v[j] = r * r;
-    }
-    stv<S, V>(out + t * F + c, v);
-  }
-}
-
 inline bool al16(const void* p) { return ((uintptr_t)p & 15) == 0; }
 
 }  // namespace
@@ -422,20 +401,5 @@ AF_EXPORT int afm_canon_conv(void* h, const void* n, const void* w,
     canon_state_kernel<<<dim3(B, (W + 255) / 256), 256, 0, s>>>(
         (float*)state, (const float*)n, (const i32*)cu, (const i32*)q_start,
         (const i32*)sslot, W, taps);
-  return af_last_err();
-}
-
-AF_EXPORT int afm_relu2(void* out, const void* z, i64 ldz, int T, int F,
-                        int dt, void* stream) {
-  if (T == 0 || F == 0) return 0;
-  hipStream_t s = (hipStream_t)stream;
-  const bool vec = F % 4 == 0 && ldz % 4 == 0 && al16(out) && al16(z);
-  const i64 total = (i64)T * (vec ? F / 4 : F);
-  const int grid = (int)((total + 255) / 256 < 16384 ? (total + 255) / 256 : 16384);
-#define R2(S, V) relu2_kernel<S, V><<<grid, 256, 0, s>>>((S*)out, (const S*)z, ldz, T, F)
-  if (dt == 0) { if (vec) R2(u16, 4); else R2(u16, 1); }
-  else if (dt == 1) { if (vec) R2(float, 4); else R2(float, 1); }
-  else return 9002;
-#undef R2
   return af_last_err();
 }

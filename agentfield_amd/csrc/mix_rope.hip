@@ -1,6 +1,7 @@
-// Row steps in front of rotary attention: the step's cos / sin table, and
-// bias, per-head RMSNorm, partial rotary positions and the K/V page append
-// in one pass over a row.
+// Row steps in front of rotary attention: the step's cos / sin table; bias,
+// per-head RMSNorm, partial rotary positions and the K/V page append in one
+// pass over a row; short causal convolutions over q, k and v, RMSNorm over the
+// whole q and k rows, rotation and page append in one pass over a row.
 //
 // Storage dtype S is bf16 (raw u16) or fp32; statistics, angles and the
 // rotation are fp32 (the table's angles double precision).
@@ -217,6 +218,247 @@ __global__ void __launch_bounds__(256) qk_rope_cache_pairs_kernel(
   }
 }
 
+// ------------------------- convolution, whole-row norm, rotation, page append
+// p [T, C] holds [q (H*dk) | k (G*dk) | v (G*dv)] per row at stride ldp.  Every
+// channel is first convolved over time (taps tap-major in cw [taps, C]; inputs
+// from before a chunk from the sequence's slot of `state` [slots, taps-1, C],
+// oldest first; inputs before position 0 are zero), then the q row and the k
+// row are RMS-normed as wholes (weights qw [H*dk], kw [G*dk]; null: no norm) and
+// the first `rot` dims of every head are rotated (dim i with i + rot/2, the
+// row's cos | sin in tab).  q goes to a contiguous [T, H*dk] buffer, k and v to
+// their pages.  STEP: every chunk is one row, and the slot moves on to the last
+// taps-1 inputs here.
+struct ConvRopeArgs {
+  const i32 *row_seq, *cu, *q_start, *sslot;
+  const float* tab;
+  const i64* slots;
+  i64 ldp;
+  float eps;
+  int T, H, G, dk, dv, rot, page, taps, rows;
+};
+
+// One row per workgroup, any sizes.  LDS: the convolved q and k rows wait in
+// LDS for the norm; otherwise they are evaluated again.
+template <typename S, bool STEP, bool LDS>
+__global__ void __launch_bounds__(256) conv_qk_rope_kernel(
+    S* __restrict__ qo, const S* __restrict__ p, const S* __restrict__ cw,
+    S* state, const S* __restrict__ qw, const S* __restrict__ kw,
+    S* __restrict__ kc, S* __restrict__ vc, ConvRopeArgs A) {
+  extern __shared__ float buf[];           // [nq + nk]
+  __shared__ float red[8];
+  const int nq = A.H * A.dk, nk = A.G * A.dk, nv = A.G * A.dv, C = nq + nk + nv;
+  const int t = blockIdx.x, b = A.row_seq[t];
+  const int k = t - A.cu[b], pos = A.q_start[b] + k;
+  const int hist = A.taps - 1;
+  S* st = state + (size_t)A.sslot[b] * hist * C;
+  auto conv = [&](int c) {
+    float acc = 0.f;
+    for (int l = 0; l <= hist; ++l) {      // lag
+      if (pos - l < 0) break;
+      const float v = l <= k ? ldf<S>(p + (size_t)(t - l) * A.ldp + c)
+                             : ldf<S>(st + (size_t)(hist - (l - k)) * C + c);
+      acc += ldf<S>(cw + (size_t)(hist - l) * C + c) * v;
+    }
+    return acc;
+  };
+  float sq = 0.f, sk = 0.f;
+  for (int c = threadIdx.x; c < nq + nk; c += 256) {
+    const float v = conv(c);
+    if (LDS) buf[c] = v;
+    (c < nq ? sq : sk) += v * v;
+  }
+  sq = wave_sum_f32(sq);
+  sk = wave_sum_f32(sk);
+  if ((threadIdx.x & 63) == 0) {
+    red[threadIdx.x >> 6] = sq;
+    red[4 + (threadIdx.x >> 6)] = sk;
+  }
+  __syncthreads();
+  const float rq = qw ? 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)nq + A.eps) : 1.f;
+  const float rk = kw ? 1.0f / sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)nk + A.eps) : 1.f;
+  auto normed = [&](int c) {
+    const float v = LDS ? buf[c] : conv(c);
+    if (c < nq) return qw ? v * rq * ldf<S>(qw + c) : v;
+    return kw ? v * rk * ldf<S>(kw + c - nq) : v;
+  };
+  const float* cs = A.tab + (size_t)t * A.rot;  // [half] cos, [half] sin
+  const int half = A.rot / 2;
+  const i64 sl = A.slots[t];
+  const i64 pg = sl / A.page, off = sl % A.page;
+  for (int c = threadIdx.x; c < nq + nk; c += 256) {
+    const int e = c < nq ? c : c - nq;
+    const int d = e % A.dk;
+    float x = normed(c);
+    if (d < half) x = x * cs[d] - normed(c + half) * cs[half + d];
+    else if (d < A.rot) x = x * cs[d - half] + normed(c - half) * cs[d];
+    if (c < nq) stf<S>(qo + (size_t)t * nq + c, x);
+    else if (sl >= 0)
+      stf<S>(kc + (((size_t)pg * A.G + e / A.dk) * A.page + off) * A.dk + d, x);
+  }
+  if (sl >= 0)
+    for (int e = threadIdx.x; e < nv; e += 256)
+      stf<S>(vc + (((size_t)pg * A.G + e / A.dv) * A.page + off) * A.dv + e % A.dv,
+             conv(nq + nk + e));
+  if (STEP && hist > 0) {
+    __syncthreads();                       // every thread has read the slot
+    for (int c = threadIdx.x; c < C; c += 256)
+      for (int j = 0; j < hist; ++j) {     // entry j: position pos - hist + 1 + j
+        S v = S(0);
+        if (pos - hist + 1 + j >= 0)
+          v = j == hist - 1 ? p[(size_t)t * A.ldp + c] : st[(size_t)(j + 1) * C + c];
+        st[(size_t)j * C + c] = v;
+      }
+  }
+}
+
+__device__ __forceinline__ short bf_bits(float f) {   // hardware rounding
+  return __builtin_bit_cast(short, static_cast<__bf16>(f));
+}
+
+// bf16 rows whose sizes are multiples of 4 (rot of 8): a thread owns NG groups
+// of four channels over A.rows consecutive rows, so its taps, norm weights and
+// the inputs behind the current row sit in registers; the next row is loaded
+// while the current one is reduced and rotated.  The convolved rows times the
+// norm weights meet their rotation partners in LDS, two rows in turn, which
+// leaves one barrier a row.
+template <int TAPS, int NG, int NT, bool STEP>
+__global__ void __launch_bounds__(NT) conv_qk_rope_bf16_kernel(
+    u16* __restrict__ qo, const u16* __restrict__ p, const u16* __restrict__ cw,
+    u16* state, const u16* __restrict__ qw, const u16* __restrict__ kw,
+    u16* __restrict__ kc, u16* __restrict__ vc, ConvRopeArgs A) {
+  constexpr int HIST = TAPS - 1, NW = NT / 64;
+  extern __shared__ __align__(16) float buf2[];      // [2][nq + nk]
+  __shared__ float red[2][2][NW];
+  const int nq = A.H * A.dk, nk = A.G * A.dk, nv = A.G * A.dv, nqk = nq + nk;
+  const int C = nqk + nv, half = A.rot / 2;
+  const int t0 = blockIdx.x * A.rows, t1 = min(A.T, t0 + A.rows);
+  auto get = [](const u16* q) { return *reinterpret_cast<const s16x4*>(q); };
+  const s16x4 zero = {0, 0, 0, 0}, one = {0x3f80, 0x3f80, 0x3f80, 0x3f80};
+
+  s16x4 wt[NG][TAPS], hist[NG][HIST > 0 ? HIST : 1], nw[NG], cur[NG], nxt[NG];
+  int dd[NG];            // dim inside the head
+  int po[NG];            // k, v: head * page * dim + dim inside the page
+#pragma unroll
+  for (int g = 0; g < NG; ++g) {
+    const int c = (g * NT + threadIdx.x) * 4;
+    nw[g] = one;
+    cur[g] = nxt[g] = zero;
+    dd[g] = po[g] = 0;
+    if (c >= C) continue;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) wt[g][j] = get(cw + (size_t)j * C + c);
+    if (c < nq) {
+      if (qw) nw[g] = get(qw + c);
+      dd[g] = c % A.dk;
+    } else if (c < nqk) {
+      if (kw) nw[g] = get(kw + c - nq);
+      dd[g] = (c - nq) % A.dk;
+      po[g] = (c - nq) / A.dk * A.page * A.dk + dd[g];
+    } else {
+      const int e = c - nqk;
+      po[g] = e / A.dv * A.page * A.dv + e % A.dv;
+    }
+    nxt[g] = get(p + (size_t)t0 * A.ldp + c);
+  }
+  for (int t = t0; t < t1; ++t) {
+    const int b = A.row_seq[t];
+    const int k = t - A.cu[b], pos = A.q_start[b] + k;
+    u16* st = state + (size_t)A.sslot[b] * HIST * C;
+    const i64 sl = A.slots[t];
+    const i64 pg = sl / A.page, off = sl % A.page;
+    float* row = buf2 + (size_t)((t - t0) & 1) * nqk;
+    if (t == t0 || k == 0) {               // the inputs behind this row
+#pragma unroll
+      for (int g = 0; g < NG; ++g) {
+        const int c = (g * NT + threadIdx.x) * 4;
+        if (c >= C) continue;
+#pragma unroll
+        for (int l = 1; l <= HIST; ++l)
+          hist[g][l - 1] = pos - l < 0 ? zero
+              : l <= k ? get(p + (size_t)(t - l) * A.ldp + c)
+                       : get(st + (size_t)(HIST - (l - k)) * C + c);
+      }
+    }
+    float acc[NG][4];
+    float sq = 0.f, sk = 0.f;
+#pragma unroll
+    for (int g = 0; g < NG; ++g) {
+      const int c = (g * NT + threadIdx.x) * 4;
+      cur[g] = nxt[g];
+      if (c >= C) continue;
+      if (t + 1 < t1) nxt[g] = get(p + (size_t)(t + 1) * A.ldp + c);
+      float ss = 0.f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        float a = bf2f((u16)wt[g][HIST][j]) * bf2f((u16)cur[g][j]);
+#pragma unroll
+        for (int l = 1; l <= HIST; ++l)
+          a += bf2f((u16)wt[g][HIST - l][j]) * bf2f((u16)hist[g][l - 1][j]);
+        ss += a * a;
+        acc[g][j] = a;
+      }
+      if (c < nqk) {
+        (c < nq ? sq : sk) += ss;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[g][j] *= bf2f((u16)nw[g][j]);
+        *reinterpret_cast<f32x4*>(row + c) = f32x4{acc[g][0], acc[g][1], acc[g][2], acc[g][3]};
+      } else if (sl >= 0) {
+        const s16x4 o = {bf_bits(acc[g][0]), bf_bits(acc[g][1]), bf_bits(acc[g][2]), bf_bits(acc[g][3])};
+        *reinterpret_cast<s16x4*>(vc + (size_t)pg * A.G * A.page * A.dv + po[g] + off * A.dv) = o;
+      }
+      if (STEP) {
+#pragma unroll
+        for (int j = 0; j < HIST; ++j)     // entry j keeps lag HIST - 1 - j
+          *reinterpret_cast<s16x4*>(st + (size_t)j * C + c) =
+              j == HIST - 1 ? cur[g] : hist[g][HIST - 2 - j];
+      } else if (HIST > 0) {
+#pragma unroll
+        for (int l = HIST - 1; l > 0; --l) hist[g][l] = hist[g][l - 1];
+        hist[g][0] = cur[g];
+      }
+    }
+    sq = wave_sum_f32(sq);
+    sk = wave_sum_f32(sk);
+    float(*rd)[NW] = red[(t - t0) & 1];
+    if ((threadIdx.x & 63) == 0) {
+      rd[0][threadIdx.x >> 6] = sq;
+      rd[1][threadIdx.x >> 6] = sk;
+    }
+    // the other buffer's readers are all past their row once this is passed
+    __syncthreads();
+    float rq = 1.f, rk = 1.f;
+    {
+      float a = 0.f, e = 0.f;
+#pragma unroll
+      for (int i = 0; i < NW; ++i) { a += rd[0][i]; e += rd[1][i]; }
+      if (qw) rq = 1.0f / sqrtf(a / (float)nq + A.eps);
+      if (kw) rk = 1.0f / sqrtf(e / (float)nk + A.eps);
+    }
+    const float* cs = A.tab + (size_t)t * A.rot;
+#pragma unroll
+    for (int g = 0; g < NG; ++g) {
+      const int c = (g * NT + threadIdx.x) * 4;
+      if (c >= nqk) continue;
+      const int d = dd[g];
+      if (d < A.rot) {
+        const bool low = d < half;
+        const f32x4 co = *reinterpret_cast<const f32x4*>(cs + (low ? d : d - half));
+        const f32x4 si = *reinterpret_cast<const f32x4*>(cs + (low ? half + d : d));
+        const f32x4 y = *reinterpret_cast<const f32x4*>(row + (low ? c + half : c - half));
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          acc[g][j] = acc[g][j] * co[j] + (low ? -y[j] : y[j]) * si[j];
+      }
+      const float rs = c < nq ? rq : rk;
+      const s16x4 o = {bf_bits(acc[g][0] * rs), bf_bits(acc[g][1] * rs),
+                       bf_bits(acc[g][2] * rs), bf_bits(acc[g][3] * rs)};
+      if (c < nq) *reinterpret_cast<s16x4*>(qo + (size_t)t * nq + c) = o;
+      else if (sl >= 0)
+        *reinterpret_cast<s16x4*>(kc + (size_t)pg * A.G * A.page * A.dk + po[g] + off * A.dk) = o;
+    }
+  }
+}
+
 }  // namespace
 
 AF_EXPORT int afm_rotary_table(void* tab, const void* positions,
@@ -264,5 +506,72 @@ AF_EXPORT int afm_qk_rope_cache(
   else MIX_DISPATCH(dt, (QRC(u16, false)), (QRC(float, false)));
 #undef QRP
 #undef QRC
+  return af_last_err();
+}
+
+// p [T, H*dk + G*dk + G*dv] at row stride ldp; state (or null when taps is 1)
+// [slots, taps-1, H*dk + G*dk + G*dv]; step: every chunk is one row and the
+// slots move on, otherwise the caller moves them (afm_conv_state).
+AF_EXPORT int afm_conv_qk_rope_cache(
+    void* qo, const void* p, i64 ldp, const void* cw, int taps, void* state,
+    const void* row_seq, const void* cu, const void* q_start,
+    const void* sslot, const void* qw, const void* kw, const void* tab,
+    int rot, void* kc, void* vc, const void* slots, float eps, int T, int H,
+    int G, int dk, int dv, int page, int step, int dt, void* stream) {
+  if (T == 0) return 0;
+  if (H < 1 || G < 1 || dk < 1 || dv < 1 || taps < 1) return 9003;
+  if (taps > 1 && !state) return 9003;
+  if (rot < 0 || rot > dk || rot % 2 != 0 || (rot > 0 && !tab)) return 9003;
+  const int nq = H * dk, nk = G * dk, nv = G * dv, C = nq + nk + nv;
+  if (ldp < C) return 9003;
+  hipStream_t s = (hipStream_t)stream;
+  ConvRopeArgs A{(const i32*)row_seq, (const i32*)cu, (const i32*)q_start,
+                 (const i32*)sslot, (const float*)tab, (const i64*)slots, ldp,
+                 eps, T, H, G, dk, dv, rot, page, taps, 1};
+  auto al = [](const void* q, size_t n) { return (uintptr_t)q % n == 0; };
+  const size_t sm2 = (size_t)2 * (nq + nk) * sizeof(float);
+  const int groups = (C + 3) / 4;
+  const int nt = step ? 1024 : 256, ng = (groups + nt - 1) / nt;
+  const bool fast = dt == 0 && taps <= 4 && ng <= (step ? 2 : 8) &&
+      dk % 4 == 0 && dv % 4 == 0 && ldp % 4 == 0 && rot % 8 == 0 &&
+      sm2 <= 60000 && al(p, 8) && al(qo, 8) && al(cw, 8) && al(state, 8) &&
+      al(qw, 8) && al(kw, 8) && al(kc, 8) && al(vc, 8) && al(tab, 16);
+  if (fast) {
+    if (!step) A.rows = T >= 8192 ? 8 : T >= 2048 ? 4 : T >= 512 ? 2 : 1;
+    const int grid = (T + A.rows - 1) / A.rows;
+#define CQF(TP, NG, NT, SP)                                                  \
+  conv_qk_rope_bf16_kernel<TP, NG, NT, SP><<<grid, NT, sm2, s>>>((u16*)qo,   \
+      (const u16*)p, (const u16*)cw, (u16*)state, (const u16*)qw,            \
+      (const u16*)kw, (u16*)kc, (u16*)vc, A)
+#define CQN(TP)                                                              \
+  do {                                                                       \
+    if (step) { if (ng <= 1) CQF(TP, 1, 1024, true); else CQF(TP, 2, 1024, true); } \
+    else if (ng <= 2) CQF(TP, 2, 256, false);                                \
+    else if (ng <= 4) CQF(TP, 4, 256, false);                                \
+    else if (ng <= 6) CQF(TP, 6, 256, false);                                \
+    else CQF(TP, 8, 256, false);                                             \
+  } while (0)
+    if (taps == 1) CQN(1);
+    else if (taps == 2) CQN(2);
+    else if (taps == 3) CQN(3);
+    else CQN(4);
+#undef CQN
+#undef CQF
+    return af_last_err();
+  }
+  const size_t sm = (size_t)(nq + nk) * sizeof(float);
+  const bool lds = sm <= 60000;
+#define CQ(ST, SP, L)                                                        \
+  conv_qk_rope_kernel<ST, SP, L><<<T, 256, L ? sm : 0, s>>>((ST*)qo,         \
+      (const ST*)p, (const ST*)cw, (ST*)state, (const ST*)qw, (const ST*)kw, \
+      (ST*)kc, (ST*)vc, A)
+#define CQL(ST)                                                              \
+  do {                                                                       \
+    if (step) { if (lds) CQ(ST, true, true); else CQ(ST, true, false); }     \
+    else { if (lds) CQ(ST, false, true); else CQ(ST, false, false); }        \
+  } while (0)
+  MIX_DISPATCH(dt, CQL(u16), CQL(float));
+#undef CQL
+#undef CQ
   return af_last_err();
 }

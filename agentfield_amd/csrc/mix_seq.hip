@@ -203,11 +203,11 @@ __global__ void __launch_bounds__(256) masked_attention_kernel(
     }
     return;
   }
-  const float inv = 1.0f / l;
+  const float inv = attn_head_gate<S>(ex, t, h) / l;
 #pragma unroll
   for (int i = 0; i < MAXV; ++i) {
     const int d = lane + 64 * i;
-    if (d < dv) stf<S>(out + ((size_t)t * H + h) * dv + d, acc[i] * inv);
+    if (d < dv) stf<S>(out + (size_t)t * ex.ldo + (size_t)h * dv + d, acc[i] * inv);
   }
 }
 
@@ -432,7 +432,8 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(
 #pragma unroll
     for (int w = 0; w < 4; ++w) o += red[(w * GQ + gg) * dvp + d];
     if (!part_o)
-      stf<S>(out + ((size_t)t * H + h0 + gg) * dv + d, o / l_run[gg]);
+      stf<S>(out + (size_t)t * ex.ldo + (size_t)(h0 + gg) * dv + d,
+             o / l_run[gg] * attn_head_gate<S>(ex, t, h0 + gg));
     else
       part_o[(((size_t)t * H + h0 + gg) * nsplit + sp) * dv + d] = o;
   }
@@ -449,16 +450,19 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(
 template <typename S>
 __global__ void __launch_bounds__(256) attn_split_combine_kernel(
     S* __restrict__ out, const float* __restrict__ part_o,
-    const float* __restrict__ part_ml, int n_rh, int nsplit, int dv) {
+    const float* __restrict__ part_ml, int n_rh, int H, int nsplit, int dv,
+    AttnExtra ex) {
   const int rh = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (rh >= n_rh) return;
+  const int t = rh / H, h = rh % H;
   const int lane = threadIdx.x & 63;
   const float* ml = part_ml + (size_t)rh * nsplit * 2;
   const float ms = lane < nsplit ? ml[2 * lane] : AF_NEG_INF;
   const float ls = lane < nsplit ? ml[2 * lane + 1] : 0.f;
   const float m = wave_max_f32(ms);
   const float w = ms > AF_NEG_INF ? expf(ms - m) : 0.f;
-  const float inv = 1.0f / wave_sum_f32(w * ls);
+  const float inv = attn_head_gate<S>(ex, t, h) / wave_sum_f32(w * ls);
+  S* orow = out + (size_t)t * ex.ldo + (size_t)h * dv;
   for (int d0 = 0; d0 < dv; d0 += 64) {
     const int d = d0 + lane;
     float o = 0.f;
@@ -467,7 +471,7 @@ __global__ void __launch_bounds__(256) attn_split_combine_kernel(
       if (ws > 0.f && d < dv)
         o += part_o[((size_t)rh * nsplit + s) * dv + d] * ws;
     }
-    if (d < dv) stf<S>(out + (size_t)rh * dv + d, o * inv);
+    if (d < dv) stf<S>(orow + d, o * inv);
   }
 }
 
@@ -799,7 +803,7 @@ static int launch_attention(void* out, const void* q, const void* kc,
 #undef ROWS
     if (nsplit > 1 && out)
       attn_split_combine_kernel<S><<<(T * H + 3) / 4, 256, 0, s>>>(
-          (S*)out, part_o, part_ml, T * H, nsplit, dv);
+          (S*)out, part_o, part_ml, T * H, H, nsplit, dv, ex);
     return af_last_err();
   }
   // very wide heads: one wave per (row, head), scalar key walk, no key splits
@@ -829,8 +833,9 @@ AF_EXPORT int afm_masked_attention(
     int G, int dk, int dv, int page, int maxp, int chunk, int window, i64 ldq,
     int nsplit, void* part_o, void* part_ml, const void* sink, float cap,
     const void* r1, const void* r2, i64 ldv, int keep_first, int vshare,
-    int dt, void* stream) {
+    const void* gate, i64 ldg, i64 ldo, int dt, void* stream) {
   if (T == 0) return 0;
+  if (out && (ldo < (i64)H * dv || (gate && ldg < H))) return 9003;
   if (G <= 0 || H % G || dv > 1024 || dk > 2048) return 9003;
   if (vshare < 1 || G % vshare) return 9003;
   if (nsplit < 1 || nsplit > 64 ||
@@ -838,7 +843,7 @@ AF_EXPORT int afm_masked_attention(
   if (ldv < dv || cap < 0.f || ((r1 == nullptr) != (r2 == nullptr))) return 9003;
   if (keep_first < 0) return 9003;
   const AttnExtra ex{(const float*)sink, (const float*)r1, (const float*)r2,
-                     cap, ldv, keep_first, vshare};
+                     cap, ldv, keep_first, vshare, gate, ldg, ldo};
   hipStream_t s = (hipStream_t)stream;
   if (dt == 0)
     return launch_attention<u16>(out, q, kc, vc, bt, row_seq, positions, scale,
@@ -886,19 +891,27 @@ AF_EXPORT int afm_diff_combine(void* out, const void* part_o,
   return af_last_err();
 }
 
-// out [T*H, dv] bf16 from part_o [T*H, nsplit, dv] / part_ml [T*H, nsplit, 2].
+// out [T, H*dv] at row stride ldo from part_o [T, H, nsplit, dv] / part_ml [T,
+// H, nsplit, 2]; gate [T, H] logits at row stride ldg, or null.
 AF_EXPORT int afm_attn_split_combine(void* out, const void* part_o,
-                                     const void* part_ml, int n_rh, int nsplit,
-                                     int dv, int dt, void* stream) {
-  if (n_rh == 0) return 0;
-  if (nsplit < 1 || nsplit > 64) return 9003;
+                                     const void* part_ml, int T, int H,
+                                     int nsplit, int dv, const void* gate,
+                                     i64 ldg, i64 ldo, int dt, void* stream) {
+  if (T == 0) return 0;
+  if (nsplit < 1 || nsplit > 64 || H < 1) return 9003;
+  if (ldo < (i64)H * dv || (gate && ldg < H)) return 9003;
+  const int n_rh = T * H;
+  AttnExtra ex{};
+  ex.gate = gate;
+  ex.ldg = ldg;
+  ex.ldo = ldo;
   hipStream_t s = (hipStream_t)stream;
   if (dt == 0)
     attn_split_combine_kernel<u16><<<(n_rh + 3) / 4, 256, 0, s>>>(
-        (u16*)out, (const float*)part_o, (const float*)part_ml, n_rh, nsplit, dv);
+        (u16*)out, (const float*)part_o, (const float*)part_ml, n_rh, H, nsplit, dv, ex);
   else if (dt == 1)
     attn_split_combine_kernel<float><<<(n_rh + 3) / 4, 256, 0, s>>>(
-        (float*)out, (const float*)part_o, (const float*)part_ml, n_rh, nsplit, dv);
+        (float*)out, (const float*)part_o, (const float*)part_ml, n_rh, H, nsplit, dv, ex);
   else
     return 9002;
   return af_last_err();

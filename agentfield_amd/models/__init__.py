@@ -4,6 +4,7 @@ from .zudisun import ZUDISUN_CONFIGS, ZudisunConfig, ZudisunForCausalLM
 from .fugevik import FUGEVIK_CONFIGS, FugevikConfig, FugevikForCausalLM
 from .vabedra import VABEDRA_CONFIGS, VabedraConfig, VabedraForCausalLM
 from .fironex import FIRONEX_CONFIGS, FironexConfig, FironexForCausalLM
+from .sadupel import SADUPEL_CONFIGS, SadupelConfig, SadupelForCausalLM
 from .registry import (architecture_of, build_model, load_model,
                        register_architecture)
 
@@ -14,11 +15,13 @@ CONFIGS.update(ZUDISUN_CONFIGS)
 CONFIGS.update(FUGEVIK_CONFIGS)
 CONFIGS.update(VABEDRA_CONFIGS)
 CONFIGS.update(FIRONEX_CONFIGS)
+CONFIGS.update(SADUPEL_CONFIGS)
 
 __all__ = ["LlamaConfig", "LlamaForCausalLM", "ReperaxConfig",
            "ReperaxForCausalLM", "ZudisunConfig",
            "ZudisunForCausalLM", "FugevikConfig", "FugevikForCausalLM",
            "VabedraConfig", "VabedraForCausalLM",
            "FironexConfig", "FironexForCausalLM",
+           "SadupelConfig", "SadupelForCausalLM",
            "CONFIGS", "architecture_of", "build_model",
            "load_model", "register_architecture"]

@@ -222,9 +222,9 @@ class HybridCache:
                [P, G, page, dv] in the model dtype (dv 0: key pages only,
                for layers whose values are part of the key rows; kv_heads may
                be a pair (key heads, value heads))
-      "state": {name: (shape, "f32" | "model")} - per-sequence tensors
-               [slots, *shape] (recurrent matrices, token-shift rows,
-               convolution inputs, ...)
+      "state": {name: (shape, "f32" | "i32" | "model")} - per-sequence
+               tensors [slots, *shape] (recurrent matrices, token-shift rows,
+               convolution inputs, token ids, ...)
 
     Pages live in `k[run]` / `v[run]`, state in `state[name][run]` (`rec` and
     `shift` are the names the linear-recurrence layers use).  Page 0 and slot
@@ -250,7 +250,8 @@ class HybridCache:
             for name, (shape, kind) in (need.get("state") or {}).items():
                 self.state.setdefault(name, {})[r] = torch.zeros(
                     num_slots, *shape, device=device,
-                    dtype=torch.float32 if kind == "f32" else dtype)
+                    dtype={"f32": torch.float32,
+                           "i32": torch.int32}.get(kind, dtype))
         self.rec = self.state.get("rec", {})
         self.shift = self.state.get("shift", {})
 
@@ -274,7 +275,7 @@ class HybridCache:
         n = 0
         for need in layout:
             for shape, kind in (need.get("state") or {}).values():
-                n += math.prod(shape) * (4 if kind == "f32" else itemsize)
+                n += math.prod(shape) * (itemsize if kind == "model" else 4)
         return n
 
 

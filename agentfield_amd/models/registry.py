@@ -97,6 +97,12 @@ def _load_fironex(path, device="cpu", dtype=None, **kw):
                         max_position=kw.get("max_position"))
 
 
+def _load_sadupel(path, device="cpu", dtype=None, **kw):
+    from .sadupel import load_sadupel
+    return load_sadupel(path, device=device, dtype=dtype,
+                        max_position=kw.get("max_position"))
+
+
 register_architecture(["LlamaForCausalLM", "MistralForCausalLM",
                        "MixtralForCausalLM"], _load_llama)
 register_architecture("Reperax", _load_reperax)
@@ -104,3 +110,4 @@ register_architecture("Zudisun", _load_zudisun)
 register_architecture("Fugevik", _load_fugevik)
 register_architecture("Vabedra", _load_vabedra)
 register_architecture("Fironex", _load_fironex)
+register_architecture("Sadupel", _load_sadupel)

@@ -80,10 +80,19 @@ class RoutedSpec:
     groups: int = 0             # 0: no group limit
     keep: int = 0
     shared_ff: int = 0          # 0: no shared expert
-    act: str = "silu"           # "clamped": bounded unit, see ops.glu
+    act: str = "silu"           # "clamped": bounded unit, see ops.glu;
+                                # "relu2": no gate, W_down max(W_up h, 0)^2
     limit: float = 0.0          # bound of the "clamped" unit
     score: str = "sigmoid"      # or "softmax" over all experts
     renorm: bool = True         # weights divided by the chosen scores' sum
+    group_top: int = 2          # a group scores the sum of so many experts
+    identity: int = 0           # router outputs behind the experts whose
+                                # output is the input itself
+
+    @property
+    def unit(self) -> int:
+        """Rows of one expert's input matrix."""
+        return self.ff if self.act == "relu2" else 2 * self.ff
 
 
 @dataclass
@@ -310,36 +319,90 @@ class GluMLP(nn.Module):
 
 
 class RoutedExperts(nn.Module):
-    """Mixture of gated experts behind a sigmoid or softmax router
-    (ops.moe_route) with an optional shared expert.  All gate/up weights sit in one matrix
-    [E*2F + 2Fs, W] (expert e: rows e*2F.., gate then up; shared last), all
-    down weights in one [W, E*F + Fs].
+    """Mixture of experts behind a sigmoid or softmax router (ops.moe_route):
+    gated units (or, act "relu2", plain ones) with an optional shared expert
+    and identity experts.  All gate/up weights sit in one matrix [E*2F + 2Fs,
+    W] (expert e: rows e*2F.., gate then up; shared last), all down weights in
+    one [W, E*F + Fs].
 
     Short steps (decode; graph-capturable) run every expert on every row:
     one gate/up GEMM, the gated unit scaled by the router weight (zero for
     experts not chosen), one down GEMM whose K axis sums experts and shared
     expert.  Longer steps sort (row, choice) pairs by expert, run each expert
-    on its rows and combine in fp32 in a fixed order."""
+    on its rows and combine in fp32 in a fixed order.
 
-    def __init__(self, spec: RoutedSpec, width: int):
+    hosted: the matrices are blocks of the caller's, which reads the same
+    input with other projections in one GEMM; it runs the short steps itself
+    (`is_static`, `route`) and hands its blocks to `run_sorted` in the longer
+    ones."""
+
+    def __init__(self, spec: RoutedSpec, width: int, hosted: bool = False):
         super().__init__()
         s = self.spec = spec
-        self.register_buffer("router", _f32(s.experts, width))
-        self.register_buffer("correction", _f32(s.experts))
-        self.gate_up = nn.Parameter(torch.empty(
-            s.experts * 2 * s.ff + 2 * s.shared_ff, width))
-        self.down = nn.Parameter(torch.empty(
-            width, s.experts * s.ff + s.shared_ff))
+        if not hosted and (s.act == "relu2" or s.identity):
+            raise ValueError("plain and identity experts run in a caller's "
+                             "matrices")
+        n = s.experts + s.identity
+        self.register_buffer("router", _f32(n, width))
+        self.register_buffer("correction", _f32(n))
+        if not hosted:
+            self.gate_up = nn.Parameter(torch.empty(
+                s.experts * 2 * s.ff + 2 * s.shared_ff, width))
+            self.down = nn.Parameter(torch.empty(
+                width, s.experts * s.ff + s.shared_ff))
+
+    @staticmethod
+    def is_static(T: int, md) -> bool:
+        return (not md.is_prefill) or T <= MOE_STATIC_ROWS
+
+    def route(self, h, dense: bool):
+        """(chosen experts [T, top], their weights, dense weights or None)."""
+        s = self.spec
+        z = sm.matmul(h.float(), self.router)
+        return sm.moe_route(z, self.correction, s.top, s.groups, s.keep,
+                            s.scale, dense=dense, score=s.score,
+                            renorm=s.renorm, group_top=s.group_top)
+
+    def run_sorted(self, h, idx, up, down):
+        """Each expert on the rows that chose it: up [E*unit, W], down [W,
+        E*F].  Returns (expert outputs in expert order, None without any; the
+        place of every (row, choice) in them, -1 for identity experts)."""
+        s = self.spec
+        E, F, U = s.experts, s.ff, s.unit
+        # (row, choice) pairs in expert order; one host round trip for sizes
+        flat = idx.flatten().long()
+        order = torch.argsort(flat, stable=True)
+        counts = torch.bincount(flat, minlength=E + s.identity).tolist()[:E]
+        pos = torch.empty_like(order, dtype=torch.int32)
+        pos[order] = torch.arange(order.numel(), dtype=torch.int32,
+                                  device=h.device)
+        n = sum(counts)
+        if s.identity:
+            pos.masked_fill_(flat >= E, -1)
+        if n == 0:
+            return None, pos
+        xs = h.index_select(0, torch.div(order[:n], s.top,
+                                         rounding_mode="floor"))
+        u = torch.empty(n, U, dtype=h.dtype, device=h.device)
+        ys = torch.empty(n, h.shape[1], dtype=h.dtype, device=h.device)
+        at = [0]
+        for c in counts:
+            at.append(at[-1] + c)
+        live = [(e, at[e], at[e + 1]) for e in range(E) if counts[e]]
+        for e, lo, hi in live:
+            sm.matmul(xs[lo:hi], up[e * U:(e + 1) * U], out=u[lo:hi])
+        a = sm.relu2(u) if s.act == "relu2" else \
+            sm.glu(u, F, s.act, limit=s.limit)
+        for e, lo, hi in live:
+            sm.matmul(a[lo:hi], down[:, e * F:(e + 1) * F], out=ys[lo:hi])
+        return ys, pos
 
     def forward(self, h, md):
         s = self.spec
         E, F, Fs = s.experts, s.ff, s.shared_ff
         T = h.shape[0]
-        z = sm.matmul(h.float(), self.router)
-        static = (not md.is_prefill) or T <= MOE_STATIC_ROWS
-        idx, wts, wd = sm.moe_route(z, self.correction, s.top, s.groups,
-                                    s.keep, s.scale, dense=static,
-                                    score=s.score, renorm=s.renorm)
+        static = self.is_static(T, md)
+        idx, wts, wd = self.route(h, static)
         if static:
             gu = sm.matmul(h, self.gate_up)
             act = torch.empty(T, E * F + Fs, dtype=h.dtype, device=h.device)
@@ -349,24 +412,7 @@ class RoutedExperts(nn.Module):
                 sm.glu(gu[:, E * 2 * F:], Fs, s.act, out=act[:, E * F:],
                        limit=s.limit)
             return sm.matmul(act, self.down), None
-        # (row, choice) pairs in expert order; one host round trip for sizes
-        flat = idx.flatten().long()
-        order = torch.argsort(flat, stable=True)
-        counts = torch.bincount(flat, minlength=E).tolist()
-        pos = torch.empty_like(order, dtype=torch.int32)
-        pos[order] = torch.arange(order.numel(), dtype=torch.int32,
-                                  device=h.device)
-        xs = h.index_select(0, torch.div(order, s.top, rounding_mode="floor"))
-        ys = torch.empty(T * s.top, h.shape[1], dtype=h.dtype, device=h.device)
-        o = 0
-        for e, n in enumerate(counts):
-            if n == 0:
-                continue
-            a = sm.glu(sm.matmul(xs[o:o + n],
-                                 self.gate_up[e * 2 * F:(e + 1) * 2 * F]),
-                       F, s.act, limit=s.limit)
-            ys[o:o + n] = sm.matmul(a, self.down[:, e * F:(e + 1) * F])
-            o += n
+        ys, pos = self.run_sorted(h, idx, self.gate_up, self.down)
         shared = None
         if Fs > 0:
             a = sm.glu(sm.matmul(h, self.gate_up[E * 2 * F:]), Fs, s.act,

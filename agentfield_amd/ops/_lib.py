@@ -127,12 +127,17 @@ def _mix_sigs() -> dict:
     return {
         "glue": {
             "afm_embed": [p, p, p, p, f, i, i, i, p],
+            "afm_embed_pairs": [p, p, p, p, p, p, p, p, p, i64, i64, i64, i,
+                                i, i, i, i, p],
             "afm_add_rows": [p, p, p, i, i, p],
             "afm_dual_norm_shift": [p, p, p, p, p, p, p, p, p, p, p, p, p, f,
                                     i, i, i, p],
             "afm_scatter_state": [p, p, p, p, i, i, p],
             "afm_norm_rows": [p, p, p, p, f, i, i, i, i, i, p],
             "afm_sandwich_norm": [p, p, p, i64, i, p, p, f, f, i, i, i, p],
+            "afm_residual_norm": [p, p, p, i64, p, p, p, i, p, p, i64, i, f,
+                                  p, p, f, i, i, i, p],
+            "afm_relu2": [p, i64, p, i64, p, i64, i, i, i, i, i, p],
             "afm_xielu": [p, p, i64, p, i, i, i, p],
             "afm_headnorm_gate": [p, p, p, p, f, i, i, i, i64, i, i, p],
             "afm_polynorm": [p, p, p, f, i, i, i64, i, p],
@@ -143,32 +148,34 @@ def _mix_sigs() -> dict:
             "afm_norm_residual": [p, p, p, i64, i, p, p, f, i, i, i, p],
             "afm_glu": [p, i64, i64, p, p, i64, i64, i, p, p, p, i64, i, i,
                         f, i, p],
-            "afm_moe_route": [p, p, p, p, p, i, i, i, i, i, f, i, i, p],
-            "afm_moe_combine": [p, p, p, p, p, i, i, i, i, p],
+            "afm_moe_route": [p, p, p, p, p, i, i, i, i, i, f, i, i, i, p],
+            "afm_moe_combine": [p, p, p, p, p, p, p, i64, i, i, i, i, i, p],
         },
         "seq": {
             "afm_qk_norm_cache": [p, p, p, p, p, p, p, p, p, f, i, i, i, i, i,
                                   i, i, i, i64, i64, i64, i, p],
             "afm_masked_attention": [p, p, p, p, p, p, p, f, i, i, i, i, i, i,
                                      i, i, i, i64, i, p, p, p, f, p, p, i64,
-                                     i, i, i, p],
+                                     i, i, p, i64, i64, i, p],
             "afm_diff_combine": [p, p, p, p, i64, f, f, f, i, i, i, i, i, i,
                                  p],
             "afm_attn_prefill_mfma": [p, p, p, p, p, p, p, p, p, f, i, i, i, i,
                                       i, i, i, i, i, i64, p, f, p, p, i64, i,
-                                      i, p],
+                                      i, p, i64, i64, p],
             "afm_diff_prefill_mfma": [p, p, p, p, p, p, p, p, p, f, i, i, i, i,
                                       i, i, i, i, i64, p, i64, f, f, f, p],
             "afm_attn_heads_mfma": [p, p, p, p, p, p, p, f, i, i, i, i, i, i,
                                     i, i, i, i64, i, p, p, p, f, p, p, i64, i,
-                                    i, p],
-            "afm_attn_split_combine": [p, p, p, i, i, i, i, p],
+                                    i, p, i64, i64, p],
+            "afm_attn_split_combine": [p, p, p, i, i, i, i, p, i64, i64, i,
+                                       p],
             "afm_linear_scan": [p, p, p, p, p, p, p, p, p, p, p, p, p, f, f, f,
                                 i, i, i, i, i, i64, i64, i64, i64, i, p],
         },
         "conv": {
             "afm_causal_conv": [p, p, i64, p, p, p, p, p, p, p, p, i, i, i, i,
                                 i, i, p],
+            "afm_conv_state": [p, p, i64, p, p, p, i, i, i, i, p],
         },
         "ssm": {
             "afm_selective_scan": [p, p, p, p, p, p, i64, p, i64, p, p, p, p,
@@ -187,7 +194,6 @@ def _mix_sigs() -> dict:
             "afm_hyper_step": [p, p, i64, p, p, p, p, f, p, i, i, i, i, p, p,
                                p, p, i, p, i, p],
             "afm_canon_conv": [p, p, p, p, p, p, p, p, i, i, i, i, i, p],
-            "afm_relu2": [p, p, i64, i, i, i, p],
         },
         "latent": {
             "afm_latent_prep": [p, p, p, i64, p, i64, p, p, p, f, i, i, i, i,
@@ -199,6 +205,9 @@ def _mix_sigs() -> dict:
             "afm_qk_rope_cache": [p, p, i64, p, i64, p, i64, p, p, p, p, p,
                                   p, i, p, p, p, f, i, i, i, i, i, i, i, i, i,
                                   p],
+            "afm_conv_qk_rope_cache": [p, p, i64, p, i, p, p, p, p, p, p, p,
+                                       p, i, p, p, p, f, i, i, i, i, i, i, i,
+                                       i, p],
         },
         "rglru": {
             "afm_rglru_gates": [p, p, p, p, p, p, p, i, i, i, i, p],

@@ -76,6 +76,41 @@ def embed_rows(ids: torch.Tensor, table: torch.Tensor,
     return out
 
 
+def embed_pairs(ids: torch.Tensor, table: torch.Tensor, pairs: torch.Tensor,
+                mul_prev: int, mul_cur: int, prev: torch.Tensor,
+                md) -> torch.Tensor:
+    """x[t] = table[ids[t]] + pairs[r] as an fp32 residual stream [T, W], r
+    the row of the (previous token, token) pair: (previous * mul_prev + token *
+    mul_cur) mod (rows - 1), the table's last row where a sequence starts.  The
+    token before a chunk comes from the sequence's slot of `prev` [slots, 1]
+    i32, which afterwards holds the chunk's last token."""
+    T, W = ids.numel(), table.shape[1]
+    buckets = pairs.shape[0] - 1
+    if not _gpu(table):
+        cu, qs, sl = (md.cu_seqlens.tolist(), md.q_start.tolist(),
+                      md.state_slots.tolist())
+        toks, rows = ids.tolist(), []
+        for b in range(len(qs)):
+            before = int(prev[sl[b], 0]) if qs[b] > 0 else None
+            for t in range(cu[b], cu[b + 1]):
+                rows.append(buckets if before is None else
+                            (before * mul_prev + toks[t] * mul_cur) % buckets)
+                before = toks[t]
+            if cu[b + 1] > cu[b]:
+                prev[sl[b], 0] = before
+        return table[ids.long()].float() + pairs[torch.tensor(rows)].float()
+    out = torch.empty(T, W, dtype=torch.float32, device=table.device)
+    step = not getattr(md, "is_prefill", True)
+    rc = _L().afm_embed_pairs(
+        _lib.ptr(out), _lib.ptr(table), _lib.ptr(pairs), _lib.ptr(ids),
+        _lib.ptr(prev), _lib.ptr(md.row_seq), _lib.ptr(md.cu_seqlens),
+        _lib.ptr(md.q_start), _lib.ptr(md.state_slots), int(mul_prev),
+        int(mul_cur), buckets, T, md.q_start.numel(), W, 1 if step else 0,
+        _code(table), _lib.cur_stream())
+    _lib.check(rc, "afm_embed_pairs")
+    return out
+
+
 def add_rows(x: torch.Tensor, other: torch.Tensor | None,
              vec: torch.Tensor | None) -> torch.Tensor:
     """In place x += other (same shape, fp32) + vec (one row, fp32)."""
@@ -232,7 +267,9 @@ def masked_attention(q: torch.Tensor, kcache: torch.Tensor,
                      window: int = 0, sink: torch.Tensor | None = None,
                      softcap: float = 0.0,
                      log_bias: tuple | None = None,
-                     v_width: int = 0, keep_first: int = 0) -> torch.Tensor:
+                     v_width: int = 0, keep_first: int = 0,
+                     gate: torch.Tensor | None = None,
+                     out: torch.Tensor | None = None) -> torch.Tensor:
     """Softmax attention of packed rows over the paged cache.  Row at
     position i sees key j iff j <= i, and (chunk > 0) floor(j/chunk) ==
     floor(i/chunk), and (window > 0) j > i - window; with keep_first > 0 the
@@ -244,7 +281,9 @@ def masked_attention(q: torch.Tensor, kcache: torch.Tensor,
     tanh(s / softcap); log_bias (r1, r2) [H] fp32 each: s <- s - r1[h] *
     ln(1 + r2[h] * (i - j)); sink [H] fp32: exp(sink[h]) joins the softmax
     denominator (a term without key or value, not scaled).  vcache None: the
-    values are the first v_width elements of the key rows."""
+    values are the first v_width elements of the key rows.  gate [T, H]: logits
+    whose sigmoid multiplies a head's output (may be a strided view).  out: rows
+    to write to, possibly columns of a wider buffer."""
     T = q.shape[0]
     _, G, page, dk = kcache.shape
     if vcache is None:
@@ -256,7 +295,7 @@ def masked_attention(q: torch.Tensor, kcache: torch.Tensor,
     H = heads
     r1, r2 = log_bias if log_bias is not None else (None, None)
     if not _gpu(q):
-        out = torch.zeros(T, H, dv, dtype=torch.float32)
+        res = torch.zeros(T, H, dv, dtype=torch.float32)
         qf = q.float().view(T, H, dk)
         bt = md.block_table.long()
         rs = md.row_seq.tolist()
@@ -285,12 +324,18 @@ def masked_attention(q: torch.Tensor, kcache: torch.Tensor,
             if sink is not None:
                 s = torch.cat([s, sink.float()[:, None]], 1)
             w = torch.softmax(s, -1)[:, :js.numel()]
-            out[t] = torch.einsum("hn,nhd->hd", w, vv)
-        return out.view(T, H * dv).to(q.dtype)
-    out = torch.empty(T, H * dv, dtype=q.dtype, device=q.device)
+            res[t] = torch.einsum("hn,nhd->hd", w, vv)
+        if gate is not None:
+            res *= torch.sigmoid(gate.float())[:, :, None]
+        res = res.view(T, H * dv).to(q.dtype)
+        return res if out is None else out.copy_(res)
+    if out is None:
+        out = torch.empty(T, H * dv, dtype=q.dtype, device=q.device)
     lens = getattr(md, "seq_lens", None)
+    tail = (_lib.ptr(gate), _rowstride(gate) if gate is not None else 0,
+            _rowstride(out))
     extra = (_lib.ptr(sink), float(softcap), _lib.ptr(r1), _lib.ptr(r2),
-             int(ldv), int(keep_first), 1)
+             int(ldv), int(keep_first), 1, *tail)
     if (q.dtype == torch.bfloat16 and lens is not None and dk <= 576
             and dv <= 512 and max(lens) >= MFMA_MIN_ROWS):
         # prompt portions: 64-row tiles on the matrix cores
@@ -330,8 +375,8 @@ def masked_attention(q: torch.Tensor, kcache: torch.Tensor,
             _lib.check(rc, "afm_attn_heads_mfma")
             if nsplit > 1:
                 rc = _L().afm_attn_split_combine(
-                    _lib.ptr(out), _lib.ptr(part_o), _lib.ptr(part_ml), T * H,
-                    nsplit, dv, _code(q), _lib.cur_stream())
+                    _lib.ptr(out), _lib.ptr(part_o), _lib.ptr(part_ml), T, H,
+                    nsplit, dv, *tail, _code(q), _lib.cur_stream())
                 _lib.check(rc, "afm_attn_split_combine")
             return out
     # few rows and many visible keys: cut the keys over several workgroups
@@ -426,7 +471,7 @@ def diff_attention(q: torch.Tensor, kcache: torch.Tensor,
                          device=q.device)
     part_ml = torch.empty(T, 2 * H, nsplit, 2, dtype=torch.float32,
                           device=q.device)
-    extra = (None, 0.0, None, None, dv, 0, 2)
+    extra = (None, 0.0, None, None, dv, 0, 2, None, 0, 0)
     common = (_lib.ptr(q), _lib.ptr(kcache), _lib.ptr(vcache),
               _lib.ptr(md.block_table), _lib.ptr(md.row_seq),
               _lib.ptr(positions), float(scale), T, 2 * H, G2, dk, dv, page,
@@ -619,10 +664,11 @@ def softcap(logits: torch.Tensor, cap: float) -> torch.Tensor:
     return out
 
 
-def matmul(x: torch.Tensor, w: torch.Tensor,
-           skinny: bool = True) -> torch.Tensor:
+def matmul(x: torch.Tensor, w: torch.Tensor, skinny: bool = True,
+           out: torch.Tensor | None = None) -> torch.Tensor:
     """x [M, K] @ w [N, K]^T through the vendor GEMM (hipBLASLt / rocBLAS);
-    fp32 operands run in true fp32 (no reduced-precision matrix mode).
+    fp32 operands run in true fp32 (no reduced-precision matrix mode).  out:
+    rows to write to (always the vendor GEMM).
 
     AF_MIX_SKINNY=1 sends decode-sized bf16 products (<= 64 rows, N and K
     multiples of 64) to the framework's MFMA skinny-GEMM kernel instead, with
@@ -631,6 +677,8 @@ def matmul(x: torch.Tensor, w: torch.Tensor,
     per 64-row step at width 2048, and the same tokens/s at width 4096) while
     the skinny path adds a combine launch per product, so the vendor GEMM is
     the default."""
+    if out is not None:
+        return torch.mm(x, w.t(), out=out)
     M, K = x.shape
     N = w.shape[0]
     if (skinny and _SKINNY and x.is_cuda and x.dtype == torch.bfloat16
@@ -740,14 +788,14 @@ def glu(gu: torch.Tensor, F: int, act: str,
 def moe_route(z: torch.Tensor, correction: torch.Tensor | None, top: int,
               n_groups: int = 0, keep: int = 0, scale: float = 1.0,
               dense: bool = False, score: str = "sigmoid",
-              renorm: bool = True):
+              renorm: bool = True, group_top: int = 2):
     """Router with score correction and group-limited top-k.
 
     z [T, E] fp32 logits; s = sigmoid(z) (score "softmax": softmax(z) over
     all experts); choice = s + correction.  With
     n_groups > 0 the experts form equal groups of neighbours, a group scores
-    the sum of its two largest choice scores and only experts of the `keep`
-    best groups can be chosen.  The `top` largest choice scores win; weights
+    the sum of its group_top (1 or 2) largest choice scores and only experts of
+    the `keep` best groups can be chosen.  The `top` largest choice scores win; weights
     = s / (sum of the chosen s + 1e-20) * scale (renorm False: s * scale).
     Returns (idx [T, top] i32,
     weights [T, top] fp32, dense weights [T, E] fp32 or None)."""
@@ -758,7 +806,8 @@ def moe_route(z: torch.Tensor, correction: torch.Tensor | None, top: int,
         choice = s + correction.float() if correction is not None else s.clone()
         if n_groups > 0 and keep < n_groups:
             size = E // n_groups
-            gs = choice.view(T, n_groups, size).topk(min(2, size), -1)[0].sum(-1)
+            gs = choice.view(T, n_groups, size).topk(
+                min(group_top, size), -1)[0].sum(-1)
             kept = torch.zeros(T, n_groups, dtype=torch.bool)
             kept.scatter_(1, gs.topk(keep, -1)[1], True)
             choice = choice.masked_fill(
@@ -780,33 +829,91 @@ def moe_route(z: torch.Tensor, correction: torch.Tensor | None, top: int,
                             _lib.ptr(z), _lib.ptr(correction), T, E, top,
                             int(n_groups), int(keep), float(scale),
                             1 if score == "softmax" else 0,
-                            1 if renorm else 0, _lib.cur_stream())
+                            1 if renorm else 0, int(group_top),
+                            _lib.cur_stream())
     _lib.check(rc, "afm_moe_route")
     return idx, w, wd
 
 
-def moe_combine(ys: torch.Tensor, pos: torch.Tensor, weights: torch.Tensor,
-                shared: torch.Tensor | None) -> torch.Tensor:
-    """y[t] = sum_r weights[t, r] * ys[pos[t*top + r]] (+ shared[t]), fp32,
-    summed in the order r = 0..top-1.  ys [T*top, W] holds the experts'
-    outputs in expert-sorted order, pos [T*top] i32 the place of every
-    (token, choice) in it."""
-    T, top = weights.shape
-    W = ys.shape[1]
-    if not _gpu(ys):
-        y = (ys.float()[pos.long()].view(T, top, W)
-             * weights.float()[:, :, None])
-        out = shared.float().clone() if shared is not None else \
-            torch.zeros(T, W)
+def _expert_sum(T: int, W: int, ys, pos, weights, hin, idw) -> torch.Tensor:
+    """CPU form of what the combining kernels add up: sum_r weights[t, r] *
+    ys[pos[t*top + r]] (pos < 0: nothing) + (sum_i idw[t, i]) hin[t], fp32."""
+    out = torch.zeros(T, W)
+    if ys is not None:
+        top = weights.shape[1]
+        p = pos.long().view(T, top)
+        y = torch.cat([ys.float(), torch.zeros(1, W)])[p]
         for r in range(top):
-            out += y[:, r]
-        return out
-    out = torch.empty(T, W, dtype=torch.float32, device=ys.device)
-    rc = _L().afm_moe_combine(_lib.ptr(out), _lib.ptr(ys), _lib.ptr(pos),
-                              _lib.ptr(weights), _lib.ptr(shared), T, top, W,
-                              _code(ys), _lib.cur_stream())
+            out += torch.where(p[:, r] >= 0, weights.float()[:, r],
+                               torch.zeros(()))[:, None] * y[:, r]
+    if idw is not None:
+        out += idw.float().sum(-1, keepdim=True) * hin.float()
+    return out
+
+
+def moe_combine(ys: torch.Tensor | None, pos: torch.Tensor | None,
+                weights: torch.Tensor | None, shared: torch.Tensor | None,
+                hin: torch.Tensor | None = None,
+                idw: torch.Tensor | None = None) -> torch.Tensor:
+    """y[t] = sum_r weights[t, r] * ys[pos[t*top + r]] (+ shared[t]), fp32,
+    summed in the order r = 0..top-1.  ys holds the experts' outputs in
+    expert-sorted order (None: no such terms), pos [T*top] i32 the place of
+    every (token, choice) in it, negative for choices without a row.  hin, idw
+    [T, n] fp32 (may be a strided view): + (sum_i idw[t, i]) * hin[t], experts
+    whose output is their input."""
+    ref = shared if shared is not None else ys
+    T = weights.shape[0] if weights is not None else ref.shape[0]
+    top = weights.shape[1] if ys is not None else 0
+    W = ref.shape[1]
+    if not _gpu(ref):
+        out = _expert_sum(T, W, ys, pos, weights, hin, idw)
+        return out + shared.float() if shared is not None else out
+    out = torch.empty(T, W, dtype=torch.float32, device=ref.device)
+    rc = _L().afm_moe_combine(
+        _lib.ptr(out), _lib.ptr(ys), _lib.ptr(pos), _lib.ptr(weights),
+        _lib.ptr(shared), _lib.ptr(hin), _lib.ptr(idw),
+        idw.stride(0) if idw is not None else 0,
+        idw.shape[1] if idw is not None else 0, T, top, W, _code(ref),
+        _lib.cur_stream())
     _lib.check(rc, "afm_moe_combine")
     return out
+
+
+def residual_norm(x: torch.Tensor, a: torch.Tensor | None, mult: float,
+                  w: torch.Tensor | None, eps: float, dtype: torch.dtype,
+                  vec: torch.Tensor | None = None,
+                  ys: torch.Tensor | None = None,
+                  pos: torch.Tensor | None = None,
+                  weights: torch.Tensor | None = None,
+                  hin: torch.Tensor | None = None,
+                  idw: torch.Tensor | None = None) -> torch.Tensor | None:
+    """In place on the fp32 residual: x += mult * u (+ vec), u the sum of a
+    [T, W] (or None) and of the expert terms of moe_combine; with w the next
+    input x / sqrt(mean(x^2) + eps) * w is returned in `dtype`.  vec [W] fp32 is
+    not scaled."""
+    T, W = x.shape
+    if not _gpu(x):
+        u = _expert_sum(T, W, ys, pos, weights, hin, idw)
+        if a is not None:
+            u += a.float()
+        x += mult * u
+        if vec is not None:
+            x += vec
+        if w is None:
+            return None
+        return (x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+                * w.float()).to(dtype)
+    h = torch.empty(T, W, dtype=dtype, device=x.device) \
+        if w is not None else None
+    rc = _L().afm_residual_norm(
+        _lib.ptr(x), _lib.ptr(h), _lib.ptr(a),
+        _rowstride(a) if a is not None else 0, _lib.ptr(ys), _lib.ptr(pos),
+        _lib.ptr(weights), weights.shape[1] if ys is not None else 0,
+        _lib.ptr(hin), _lib.ptr(idw), idw.stride(0) if idw is not None else 0,
+        idw.shape[1] if idw is not None else 0, float(mult), _lib.ptr(vec),
+        _lib.ptr(w), float(eps), T, W, _DT[dtype], _lib.cur_stream())
+    _lib.check(rc, "afm_residual_norm")
+    return h
 
 
 # ------------------------------------------------- selective state space
@@ -1280,14 +1387,28 @@ def gate_heads(o: torch.Tensor, gate: torch.Tensor) -> torch.Tensor:
     return out
 
 
-def relu2(z: torch.Tensor) -> torch.Tensor:
-    """max(z, 0)^2, element-wise; z [T, F] may be a strided view."""
+def relu2(z: torch.Tensor, out: torch.Tensor | None = None,
+          row_weight: torch.Tensor | None = None, unit: int = 1,
+          lead: int = 0) -> torch.Tensor:
+    """max(z, 0)^2, element-wise; z [T, F] and out may be strided views.
+    row_weight [T, >= (F - lead) / unit] fp32 (may be a strided view): the
+    columns from `lead` on form units of `unit` columns, unit e of row t is
+    multiplied by row_weight[t, e]."""
     T, F = z.shape
     if not _gpu(z):
-        return torch.relu(z.float()).pow(2).to(z.dtype)
-    out = torch.empty(T, F, dtype=z.dtype, device=z.device)
-    rc = _L().afm_relu2(_lib.ptr(out), _lib.ptr(z), _rowstride(z), T, F,
-                        _code(z), _lib.cur_stream())
+        r = torch.relu(z.float()).pow(2)
+        if row_weight is not None and F > lead:
+            n = (F - lead) // unit
+            r[:, lead:] *= row_weight[:, :n].float().repeat_interleave(unit, 1)
+        r = r.to(z.dtype)
+        return r if out is None else out.copy_(r)
+    if out is None:
+        out = torch.empty(T, F, dtype=z.dtype, device=z.device)
+    rc = _L().afm_relu2(
+        _lib.ptr(out), _rowstride(out), _lib.ptr(z), _rowstride(z),
+        _lib.ptr(row_weight),
+        row_weight.stride(0) if row_weight is not None else 0, int(lead),
+        int(unit), T, F, _code(z), _lib.cur_stream())
     _lib.check(rc, "afm_relu2")
     return out
 
@@ -1302,14 +1423,16 @@ def scaled_inv_freq(dims: int, base: float,
                     scaling: dict | None = None) -> torch.Tensor:
     """Rotary frequencies f_i = base^(-2i/dims), i < dims/2, as float64.
 
-    scaling {factor, low, high, original} rescales by wavelength l = 2 pi /
-    f: l < original/high keeps f; l > original/low gives f / factor; in
-    between, with s = (original/l - low) / (high - low), the blend (1 - s) *
-    f / factor + s * f."""
+    scaling {factor} alone divides every f by factor.  scaling {factor, low,
+    high, original} rescales by wavelength l = 2 pi / f: l < original/high
+    keeps f; l > original/low gives f / factor; in between, with s =
+    (original/l - low) / (high - low), the blend (1 - s) * f / factor + s * f."""
     out = []
     for i in range(dims // 2):
         f = float(base) ** (-2.0 * i / dims)
-        if scaling:
+        if scaling and "original" not in scaling:
+            f = f / float(scaling["factor"])
+        elif scaling:
             orig, fac = float(scaling["original"]), float(scaling["factor"])
             lo, hi = float(scaling["low"]), float(scaling["high"])
             wl = 2.0 * math.pi / f
@@ -1418,6 +1541,66 @@ def qk_rope_cache(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
         _lib.ptr(slots), float(eps), T, H, G, Gv, dk, dv, page,
         1 if pairs else 0, _code(q), _lib.cur_stream())
     _lib.check(rc, "afm_qk_rope_cache")
+    return out
+
+
+def conv_qk_rope_cache(p: torch.Tensor, conv: torch.Tensor,
+                       state: torch.Tensor, md, heads: int, kv_heads: int,
+                       eps: float, kcache: torch.Tensor, vcache: torch.Tensor,
+                       q_norm: torch.Tensor | None = None,
+                       k_norm: torch.Tensor | None = None,
+                       rot_tab: torch.Tensor | None = None) -> torch.Tensor:
+    """Row steps in front of rotary attention whose projections pass a short
+    convolution over time.  p [T, H*dk + G*dk + G*dv] (may be a strided view)
+    holds q | k | v per row; conv is tap-major [taps, channels], its last row
+    weighing the current token, the inputs before a chunk come from `state`
+    (see causal_conv).  Then RMSNorm over the whole q row and the whole k row
+    (plain weights; skipped when None), rotation of the leading rot_tab.shape[1]
+    dims of every q and k head (dim i with i + half, the rows' rotary_table),
+    and k and v go to the paged caches at md.slots.  Returns q, contiguous [T,
+    H*dk]."""
+    T, C = p.shape
+    H, G = heads, kv_heads
+    page, dk, dv = kcache.shape[2], kcache.shape[3], vcache.shape[3]
+    nq, nk = H * dk, G * dk
+    taps = conv.shape[0]
+    if C != nq + nk + G * dv or conv.shape[1] != C:
+        raise ValueError("conv_qk_rope_cache: widths do not fit the heads")
+    rot = rot_tab.shape[1] if rot_tab is not None else 0
+    if not _gpu(p):
+        u = causal_conv(p.float(), conv.float(), None, state, md, silu=False)
+
+        def normed(t, w):
+            if w is None:
+                return t
+            return t * torch.rsqrt(t.pow(2).mean(-1, keepdim=True) + eps) \
+                * w.float()
+        q = normed(u[:, :nq], q_norm).reshape(T, H, dk)
+        k = normed(u[:, nq:nq + nk], k_norm).reshape(T, G, dk)
+        if rot:
+            q, k = (rotate_rows(t, rot_tab, False) for t in (q, k))
+        pg = torch.div(md.slots, page, rounding_mode="floor")
+        off = md.slots - pg * page
+        kcache[pg, :, off] = k.to(kcache.dtype)
+        vcache[pg, :, off] = u[:, nq + nk:].reshape(T, G, dv).to(vcache.dtype)
+        return q.reshape(T, nq).to(p.dtype)
+    step = not getattr(md, "is_prefill", True)
+    B = md.q_start.numel()
+    out = torch.empty(T, nq, dtype=p.dtype, device=p.device)
+    chunks = (_lib.ptr(md.cu_seqlens), _lib.ptr(md.q_start),
+              _lib.ptr(md.state_slots))
+    rc = _L().afm_conv_qk_rope_cache(
+        _lib.ptr(out), _lib.ptr(p), _rowstride(p), _lib.ptr(conv), taps,
+        _lib.ptr(state), _lib.ptr(md.row_seq), *chunks, _lib.ptr(q_norm),
+        _lib.ptr(k_norm), _lib.ptr(rot_tab), rot, _lib.ptr(kcache),
+        _lib.ptr(vcache), _lib.ptr(md.slots), float(eps), T, H, G, dk, dv,
+        page, 1 if step else 0, _code(p), _lib.cur_stream())
+    _lib.check(rc, "afm_conv_qk_rope_cache")
+    if not step and taps > 1:
+        rc = _L().afm_conv_state(_lib.ptr(state), _lib.ptr(p), _rowstride(p),
+                                 *chunks, B, C, taps, _code(p),
+                                 _lib.cur_stream())
+        _lib.check(rc, "afm_conv_state")
     return out
 
 
