@@ -52,6 +52,7 @@ HIP_SOURCES = [
 #   conv    short depthwise causal convolution with carried inputs
 #   delta   gated delta-rule recurrence, norm after the residual sum
 #   rglru   real-gated linear recurrent unit
+#   skinny  split-K weight-streaming GEMM for few rows
 MIX_GROUPS = {
     "glue": (PKG_DIR / "libafglue.so", ["mix_glue.hip"]),
     "seq": (PKG_DIR / "libafmix.so", ["mix_seq.hip", "mix_attn_mfma.hip"]),
@@ -63,6 +64,7 @@ MIX_GROUPS = {
     "delta": (PKG_DIR / "libafdelta.so", ["mix_delta.hip"]),
     "conv": (PKG_DIR / "libafconv.so", ["mix_conv.hip"]),
     "rglru": (PKG_DIR / "libafrglru.so", ["mix_rglru.hip"]),
+    "skinny": (PKG_DIR / "libafskinny.so", ["gemm_skinny.hip"]),
 }
 MIX_SOURCES = [s for _lib, srcs in MIX_GROUPS.values() for s in srcs]
 MIX_LIB = MIX_GROUPS["seq"][0]

@@ -214,16 +214,8 @@ __global__ void __launch_bounds__(256) gemm_skinny_combine_row_kernel(
     ss_out[m * 8 + blockIdx.y] = red[0] + red[1] + red[2] + red[3];
 }
 
-AF_EXPORT int af_gemm_skinny(void* out, void* partial, void* residual,
-                             const void* X, const void* W, int M, int N,
-                             int K, int SK, int mode,
-                             const void* scale_ss, float eps, void* ss_out,
-                             void* stream) {
-  if (M < 1 || M > 256) return 9005;
-  if (N % 64 || K % 64) return 9006;
-  hipStream_t st = (hipStream_t)stream;
-  int Kc = ((K / SK + 63) / 64) * 64;
-  while ((SK - 1) * Kc >= K) --SK;  // drop empty splits
+static void launch_skinny(void* partial, const void* X, const void* W, int M,
+                          int N, int K, int SK, int Kc, hipStream_t st) {
   dim3 grid(N / 64, SK), blk(256);
   const int MT = (M + 15) / 16;
 #define AF_SK_LAUNCH(MTV)                                                      \
@@ -248,6 +240,31 @@ AF_EXPORT int af_gemm_skinny(void* out, void* partial, void* residual,
     default: AF_SK_LAUNCH(16); break;
   }
 #undef AF_SK_LAUNCH
+}
+
+// The fp32 partial sums [SK, M, N] alone, for a consumer that adds them up
+// itself: K is cut into SK pieces of Kc (a multiple of 64; none empty).
+AF_EXPORT int af_gemm_skinny_parts(void* partial, const void* X, const void* W,
+                                   int M, int N, int K, int SK, int Kc,
+                                   void* stream) {
+  if (M < 1 || M > 256) return 9005;
+  if (N % 64 || K % 64 || Kc % 64 || Kc < 64 || SK < 1) return 9006;
+  if ((i64)(SK - 1) * Kc >= K || (i64)SK * Kc < K) return 9003;
+  launch_skinny(partial, X, W, M, N, K, SK, Kc, (hipStream_t)stream);
+  return af_last_err();
+}
+
+AF_EXPORT int af_gemm_skinny(void* out, void* partial, void* residual,
+                             const void* X, const void* W, int M, int N,
+                             int K, int SK, int mode,
+                             const void* scale_ss, float eps, void* ss_out,
+                             void* stream) {
+  if (M < 1 || M > 256) return 9005;
+  if (N % 64 || K % 64) return 9006;
+  hipStream_t st = (hipStream_t)stream;
+  int Kc = ((K / SK + 63) / 64) * 64;
+  while ((SK - 1) * Kc >= K) --SK;  // drop empty splits
+  launch_skinny(partial, X, W, M, N, K, SK, Kc, st);
   if (mode == 4) {
     if (N % 32) return 9007;
     dim3 g4(M, 8);

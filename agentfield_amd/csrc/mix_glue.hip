@@ -431,9 +431,10 @@ __global__ void __launch_bounds__(256) xielu_kernel(
 
 // Residual add of a layer whose sublayers share one input, and the RMSNorm in
 // front of the next layer, in one pass over the row:
-//   u = a + sum_r wts[r] ys[pos[r]] + (sum_i idw[i]) hin
+//   u = a + sum_s parts[s] + sum_r wts[r] ys[pos[r]] + (sum_i idw[i]) hin
 //   x += mult * u (+ vec);   h = x / sqrt(mean(x^2) + eps) * w
-// a: what sits in token order (or null); ys: rows in another order, pos < 0
+// a: what sits in token order (or null); parts [np, T, W] fp32: the same as
+// partial sums of a split product (np 0: none); ys: rows in another order, pos < 0
 // skipped (top 0: none); hin: the layer's own input under the weights idw [nid]
 // at row stride ldi (nid 0: none); vec: one fp32 row; h null: no norm.
 // REG: the row fits 4 passes of the workgroup and waits in registers for the
@@ -441,10 +442,11 @@ __global__ void __launch_bounds__(256) xielu_kernel(
 template <typename S, int V, int NT, bool REG>
 __global__ void __launch_bounds__(NT) residual_norm_kernel(
     float* __restrict__ x, S* __restrict__ h, const S* __restrict__ a, i64 lda,
-    const S* __restrict__ ys, const i32* __restrict__ pos,
-    const float* __restrict__ wts, int top, const S* __restrict__ hin,
-    const float* __restrict__ idw, i64 ldi, int nid, float mult,
-    const float* __restrict__ vec, const S* __restrict__ w, float eps, int W) {
+    const float* __restrict__ parts, int np, const S* __restrict__ ys,
+    const i32* __restrict__ pos, const float* __restrict__ wts, int top,
+    const S* __restrict__ hin, const float* __restrict__ idw, i64 ldi, int nid,
+    float mult, const float* __restrict__ vec, const S* __restrict__ w,
+    float eps, int W) {
   __shared__ float red[NT / 64];
   const int t = blockIdx.x;
   float* xr = x + (size_t)t * W;
@@ -456,6 +458,12 @@ __global__ void __launch_bounds__(NT) residual_norm_kernel(
     float u[4] = {0.f, 0.f, 0.f, 0.f}, v[4];
     ldv<float, V>(xr + i, xv);
     if (a) ldv<S, V>(a + (size_t)t * lda + i, u);
+#pragma unroll 8
+    for (int s = 0; s < np; ++s) {
+      ldv<float, V>(parts + ((size_t)s * gridDim.x + t) * W + i, v);
+#pragma unroll
+      for (int j = 0; j < V; ++j) u[j] += v[j];
+    }
     for (int r = 0; r < top; ++r) {
       const int p = pr[r];
       if (p < 0) continue;
@@ -755,27 +763,33 @@ __global__ void __launch_bounds__(256) glu_kernel(
   }
 }
 
-// Sigmoid router with score correction and group-limited top-k, one wave per
-// token.  z [T, E] fp32 logits; s = sigmoid(z); choice = s + corr.  With
-// n_groups > 0 the experts form n_groups equal groups of neighbours, a
-// group's score is the sum of its two largest choice scores (gtop 1: its
-// largest choice score), and experts outside the best `keep` groups cannot be chosen.  The `top` largest choice
-// scores win (ties: lower index); weights = s / (sum of chosen s + 1e-20) *
-// scale.  Outputs idx [T, top] i32, wts [T, top] fp32 and, optionally, the
-// dense form wd [T, E] fp32 (zero for experts not chosen).
-__global__ void __launch_bounds__(64) moe_route_kernel(
-    i32* __restrict__ idx, float* __restrict__ wts, float* __restrict__ wd,
-    const float* __restrict__ z, const float* __restrict__ corr, int E,
-    int top, int n_groups, int keep, float scale, int softmax, int renorm,
-    int gtop) {
-  extern __shared__ float sh[];
+// Router with score correction and group-limited top-k of one token by one
+// wave.  zr [E] fp32 logits; s = sigmoid(z) or softmax(z) over all E; choice =
+// s + corr.  With n_groups > 0 the experts form n_groups equal groups of
+// neighbours, a group's score is the sum of its two largest choice scores (gtop
+// 1: its largest choice score), and experts outside the best `keep` groups
+// cannot be chosen.  The `top` largest choice scores win (ties: lower index);
+// weights = s / (sum of chosen s + 1e-20) * scale (renorm 0: s * scale).
+// Outputs idx [top] i32, wts [top] fp32 and, optionally, the dense form wd [E]
+// fp32 (zero for experts not chosen).  sh: 3 * E + n_groups floats of LDS that
+// belong to the wave.
+struct RouteArgs {
+  const float* corr;
+  int E, top, n_groups, keep;
+  float scale;
+  int softmax, renorm, gtop;
+};
+
+__device__ __forceinline__ void route_row(const float* zr, float* sh, i32* idx,
+                                          float* wts, float* wd,
+                                          const RouteArgs& A) {
+  const int E = A.E, lane = threadIdx.x & 63;
   float* sig = sh;             // [E]
   float* choice = sh + E;      // [E]
-  float* gsc = sh + 2 * E;     // [n_groups]
-  const int t = blockIdx.x, lane = threadIdx.x;
-  const float* zr = z + (size_t)t * E;
+  i32* list = reinterpret_cast<i32*>(sh + 2 * E);   // [top]
+  float* gsc = sh + 3 * E;     // [n_groups]
   float zmax = 0.f, zinv = 1.f;
-  if (softmax) {       // scores are softmax(z) over all experts
+  if (A.softmax) {
     zmax = -INFINITY;
     for (int e = lane; e < E; e += 64) zmax = fmaxf(zmax, zr[e]);
     zmax = wave_max_f32(zmax);
@@ -784,37 +798,36 @@ __global__ void __launch_bounds__(64) moe_route_kernel(
     zinv = 1.0f / wave_sum_f32(zs);
   }
   for (int e = lane; e < E; e += 64) {
-    const float s = softmax ? expf(zr[e] - zmax) * zinv
-                            : 1.0f / (1.0f + expf(-zr[e]));
+    const float s = A.softmax ? expf(zr[e] - zmax) * zinv
+                              : 1.0f / (1.0f + expf(-zr[e]));
     sig[e] = s;
-    choice[e] = s + (corr ? corr[e] : 0.f);
-    if (wd) wd[(size_t)t * E + e] = 0.f;
+    choice[e] = s + (A.corr ? A.corr[e] : 0.f);
   }
-  __syncthreads();
-  if (n_groups > 0 && keep < n_groups) {
-    const int size = E / n_groups;
-    for (int g = lane; g < n_groups; g += 64) {
+  __builtin_amdgcn_wave_barrier();
+  if (A.n_groups > 0 && A.keep < A.n_groups) {
+    const int size = E / A.n_groups;
+    for (int g = lane; g < A.n_groups; g += 64) {
       float a = -INFINITY, b = -INFINITY;   // largest, second largest
       for (int m = 0; m < size; ++m) {
         const float c = choice[g * size + m];
         if (c > a) { b = a; a = c; }
         else if (c > b) b = c;
       }
-      gsc[g] = size > 1 && gtop > 1 ? a + b : a;
+      gsc[g] = size > 1 && A.gtop > 1 ? a + b : a;
     }
-    __syncthreads();
-    for (int g = lane; g < n_groups; g += 64) {
+    __builtin_amdgcn_wave_barrier();
+    for (int g = lane; g < A.n_groups; g += 64) {
       const float mine = gsc[g];
       int rank = 0;
-      for (int o = 0; o < n_groups; ++o)
+      for (int o = 0; o < A.n_groups; ++o)
         rank += (gsc[o] > mine || (gsc[o] == mine && o < g)) ? 1 : 0;
-      if (rank >= keep)
+      if (rank >= A.keep)
         for (int m = 0; m < size; ++m) choice[g * size + m] = -INFINITY;
     }
-    __syncthreads();
+    __builtin_amdgcn_wave_barrier();
   }
   float total = 0.f;
-  for (int r = 0; r < top; ++r) {
+  for (int r = 0; r < A.top; ++r) {
     float bv = -INFINITY;
     int bi = 0x7fffffff;
     for (int e = lane; e < E; e += 64) {
@@ -829,18 +842,107 @@ __global__ void __launch_bounds__(64) moe_route_kernel(
     }
     if (bi >= E) bi = r < E ? r : 0;    // fewer candidates than `top`
     total += sig[bi];
+    __builtin_amdgcn_wave_barrier();
     if (lane == 0) {
-      idx[(size_t)t * top + r] = bi;
-      wts[(size_t)t * top + r] = sig[bi];
+      list[r] = bi;
       choice[bi] = -INFINITY;
     }
-    __syncthreads();
+    __builtin_amdgcn_wave_barrier();
   }
-  const float inv = renorm ? scale / (total + 1e-20f) : scale;
-  for (int r = lane; r < top; r += 64) {
-    const float w = wts[(size_t)t * top + r] * inv;
-    wts[(size_t)t * top + r] = w;
-    if (wd) wd[(size_t)t * E + idx[(size_t)t * top + r]] = w;
+  const float inv = A.renorm ? A.scale / (total + 1e-20f) : A.scale;
+  for (int e = lane; e < E; e += 64) choice[e] = 0.f;     // now the dense form
+  __builtin_amdgcn_wave_barrier();
+  for (int r = lane; r < A.top; r += 64) {
+    const int e = list[r];
+    const float w = sig[e] * inv;
+    idx[r] = e;
+    wts[r] = w;
+    choice[e] = w;
+  }
+  __builtin_amdgcn_wave_barrier();
+  if (wd)
+    for (int e = lane; e < E; e += 64) wd[e] = choice[e];
+}
+
+// One wave per token from ready logits z [T, E].
+__global__ void __launch_bounds__(64) moe_route_kernel(
+    i32* idx, float* wts, float* wd, const float* __restrict__ z, RouteArgs A) {
+  extern __shared__ float sh[];
+  const size_t t = blockIdx.x;
+  route_row(z + t * A.E, sh, idx + t * A.top, wts + t * A.top,
+            wd ? wd + t * A.E : nullptr, A);
+}
+
+// Router logits and routing of 16 tokens per workgroup of NW waves, bf16
+// inputs: z = h R^T in fp32.  Wave w takes the 32-wide steps w, w + NW, .. of
+// the inner dimension; h rows are A fragments, and the fp32 router weights
+// enter as three bf16 terms (all 24 bits), so a product is exact and only the
+// fp32 sums round.  The waves' sums meet in LDS, then wave w routes the tokens
+// w, w + NW, ..  ET: 16-expert tiles.
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+
+template <int ET, int NW>
+__global__ void __launch_bounds__(NW * 64) moe_router_kernel(
+    i32* idx, float* wts, float* wd, const u16* __restrict__ h, i64 ldh,
+    const float* __restrict__ router, int T, int W, RouteArgs A) {
+  constexpr int EP = ET * 16;
+  extern __shared__ float sh[];            // [NW][16][EP], then the waves' rows
+  const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int t0 = blockIdx.x * 16, E = A.E;
+  const u16* hr = h + (size_t)min(t0 + (lane & 15), T - 1) * ldh;
+  f32x4 acc[ET];
+#pragma unroll
+  for (int et = 0; et < ET; ++et) acc[et] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+  for (int k0 = wid * 32; k0 < W; k0 += NW * 32) {
+    const int k = k0 + (lane >> 4) * 8;    // W is a multiple of 8
+    union { s16x8 s; bf16x8 b; } a;
+    a.s = s16x8{0, 0, 0, 0, 0, 0, 0, 0};
+    if (k < W) a.s = *reinterpret_cast<const s16x8*>(hr + k);
+#pragma unroll
+    for (int et = 0; et < ET; ++et) {
+      const int n = et * 16 + (lane & 15);
+      float r[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) r[j] = 0.f;
+      if (n < E && k < W) {
+        const f32x4* rp = reinterpret_cast<const f32x4*>(router + (size_t)n * W + k);
+        const f32x4 r0 = rp[0], r1 = rp[1];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) { r[j] = r0[j]; r[4 + j] = r1[j]; }
+      }
+#pragma unroll
+      for (int term = 0; term < 3; ++term) {
+        bf16x8 b;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          b[j] = static_cast<__bf16>(r[j]);
+          r[j] -= static_cast<float>(b[j]);
+        }
+        acc[et] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.b, b, acc[et], 0, 0, 0);
+      }
+    }
+  }
+#pragma unroll
+  for (int et = 0; et < ET; ++et)
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      sh[(wid * 16 + (lane >> 4) * 4 + r) * EP + et * 16 + (lane & 15)] = acc[et][r];
+  __syncthreads();
+  float* mine = sh + NW * 16 * EP + wid * (4 * E + A.n_groups);
+  for (int row = wid; row < 16; row += NW) {
+    const size_t t = t0 + row;
+    if (t >= (size_t)T) break;
+    __builtin_amdgcn_wave_barrier();       // the previous token's row is read
+    for (int e = lane; e < E; e += 64) {
+      float z = 0.f;
+#pragma unroll
+      for (int w = 0; w < NW; ++w) z += sh[(w * 16 + row) * EP + e];
+      mine[e] = z;
+    }
+    __builtin_amdgcn_wave_barrier();
+    route_row(mine, mine + E, idx + t * A.top, wts + t * A.top,
+              wd ? wd + t * E : nullptr, A);
   }
 }
 
@@ -1126,26 +1228,28 @@ AF_EXPORT int afm_sandwich_norm(void* x, void* h, const void* y, i64 ldy,
 // x [T, W] fp32 in place; a at row stride lda, hin [T, W], ys rows of W in the
 // storage dtype; h (or null) [T, W] in the storage dtype.
 AF_EXPORT int afm_residual_norm(void* x, void* h, const void* a, i64 lda,
-                                const void* ys, const void* pos,
+                                const void* parts, int np, const void* ys, const void* pos,
                                 const void* wts, int top, const void* hin,
                                 const void* idw, i64 ldi, int nid, float mult,
                                 const void* vec, const void* w, float eps,
                                 int T, int W, int dt, void* stream) {
   if (T == 0) return 0;
   if (h && !w) return 9003;
+  if (np < 0 || (np > 0 && !parts)) return 9003;
   if (top < 0 || (top > 0 && (!ys || !pos || !wts))) return 9003;
   if (nid < 0 || (nid > 0 && (!hin || !idw))) return 9003;
   hipStream_t s = (hipStream_t)stream;
   const bool vv = W % 4 == 0 && lda % 4 == 0 &&
-                  aligned16(x, h, a, ys, hin, vec, w);
+                  aligned16(x, h, a, ys, hin, vec, w) && aligned16(parts);
   const int cols = W / (vv ? 4 : 1);
   // few rows of many columns: one column group per thread
   const bool wide = T <= 512 && cols > 256;
 #define RNK(ST, V, NT, R)                                                    \
   residual_norm_kernel<ST, V, NT, R><<<T, NT, 0, s>>>((float*)x, (ST*)h,     \
-      (const ST*)a, lda, (const ST*)ys, (const i32*)pos, (const float*)wts,  \
-      top, (const ST*)hin, (const float*)idw, ldi, nid, mult,                \
-      (const float*)vec, (const ST*)w, eps, W)
+      (const ST*)a, lda, (const float*)parts, np, (const ST*)ys,             \
+      (const i32*)pos, (const float*)wts, top, (const ST*)hin,               \
+      (const float*)idw, ldi, nid, mult, (const float*)vec, (const ST*)w,    \
+      eps, W)
 #define RNR(ST, V)                                                           \
   do {                                                                       \
     if (wide && cols <= SWN_IT * 1024) RNK(ST, V, 1024, true);               \
@@ -1246,12 +1350,42 @@ AF_EXPORT int afm_moe_route(void* idx, void* wts, void* wd, const void* z,
   if (gtop < 1 || gtop > 2) return 9003;
   if (E < 1 || top < 1 || top > E) return 9003;
   if (n_groups > 0 && (E % n_groups != 0 || keep < 1)) return 9003;
-  const size_t sm = (size_t)(2 * E + (n_groups > 0 ? n_groups : 0)) *
+  const size_t sm = (size_t)(3 * E + (n_groups > 0 ? n_groups : 0)) *
                     sizeof(float);
   if (sm > 60000) return 9004;
+  const RouteArgs A{(const float*)corr, E, top, n_groups, keep, scale, softmax,
+                    renorm, gtop};
   moe_route_kernel<<<T, 64, sm, (hipStream_t)stream>>>(
-      (i32*)idx, (float*)wts, (float*)wd, (const float*)z, (const float*)corr,
-      E, top, n_groups, keep, scale, softmax, renorm, gtop);
+      (i32*)idx, (float*)wts, (float*)wd, (const float*)z, A);
+  return af_last_err();
+}
+
+// h [T, W] bf16 at row stride ldh, router [E, W] fp32; 9004: sizes the fused
+// form does not take (the caller makes the logits itself).
+AF_EXPORT int afm_moe_router(void* idx, void* wts, void* wd, const void* h,
+                             i64 ldh, const void* router, const void* corr,
+                             int T, int W, int E, int top, int n_groups,
+                             int keep, float scale, int softmax, int renorm,
+                             int gtop, void* stream) {
+  if (T == 0) return 0;
+  if (gtop < 1 || gtop > 2) return 9003;
+  if (E < 1 || top < 1 || top > E) return 9003;
+  if (n_groups > 0 && (E % n_groups != 0 || keep < 1)) return 9003;
+  if (E > 128 || W % 8 || ldh % 8 || !aligned16(h, router)) return 9004;
+  const RouteArgs A{(const float*)corr, E, top, n_groups, keep, scale, softmax,
+                    renorm, gtop};
+  const int grid = (T + 15) / 16;
+#define MR(ET, NW)                                                           \
+  moe_router_kernel<ET, NW><<<grid, NW * 64,                                 \
+      (size_t)(NW * 16 * ET * 16 + NW * (4 * E + (n_groups > 0 ? n_groups : 0))) * \
+          sizeof(float), (hipStream_t)stream>>>(                             \
+      (i32*)idx, (float*)wts, (float*)wd, (const u16*)h, ldh,                \
+      (const float*)router, T, W, A)
+  if (E <= 16) MR(1, 16);
+  else if (E <= 32) MR(2, 16);
+  else if (E <= 64) MR(4, 8);
+  else MR(8, 4);
+#undef MR
   return af_last_err();
 }
 

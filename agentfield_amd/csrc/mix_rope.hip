@@ -315,6 +315,13 @@ __device__ __forceinline__ short bf_bits(float f) {   // hardware rounding
   return __builtin_bit_cast(short, static_cast<__bf16>(f));
 }
 
+// A barrier for data that meets in LDS: global loads and stores stay in flight.
+__device__ __forceinline__ void lds_barrier() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+}
+
 // bf16 rows whose sizes are multiples of 4 (rot of 8): a thread owns NG groups
 // of four channels over A.rows consecutive rows, so its taps, norm weights and
 // the inputs behind the current row sit in registers; the next row is loaded
@@ -322,7 +329,7 @@ __device__ __forceinline__ short bf_bits(float f) {   // hardware rounding
 // norm weights meet their rotation partners in LDS, two rows in turn, which
 // leaves one barrier a row.
 template <int TAPS, int NG, int NT, bool STEP>
-__global__ void __launch_bounds__(NT) conv_qk_rope_bf16_kernel(
+__global__ void __launch_bounds__(NT, NG <= 2 ? 4 : 2) conv_qk_rope_bf16_kernel(
     u16* __restrict__ qo, const u16* __restrict__ p, const u16* __restrict__ cw,
     u16* state, const u16* __restrict__ qw, const u16* __restrict__ kw,
     u16* __restrict__ kc, u16* __restrict__ vc, ConvRopeArgs A) {
@@ -365,7 +372,7 @@ __global__ void __launch_bounds__(NT) conv_qk_rope_bf16_kernel(
     const int k = t - A.cu[b], pos = A.q_start[b] + k;
     u16* st = state + (size_t)A.sslot[b] * HIST * C;
     const i64 sl = A.slots[t];
-    const i64 pg = sl / A.page, off = sl % A.page;
+    const uint32_t pg = (uint32_t)sl / (uint32_t)A.page, off = (uint32_t)sl % (uint32_t)A.page;
     float* row = buf2 + (size_t)((t - t0) & 1) * nqk;
     if (t == t0 || k == 0) {               // the inputs behind this row
 #pragma unroll
@@ -388,6 +395,11 @@ __global__ void __launch_bounds__(NT) conv_qk_rope_bf16_kernel(
       if (c >= C) continue;
       if (t + 1 < t1) nxt[g] = get(p + (size_t)(t + 1) * A.ldp + c);
       float ss = 0.f;
+      // the weights stay packed: unpacked for the whole loop they would take
+      // the registers of two more waves
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) asm volatile("" : "+v"(wt[g][j]));
+      asm volatile("" : "+v"(nw[g]));
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         float a = bf2f((u16)wt[g][HIST][j]) * bf2f((u16)cur[g][j]);
@@ -425,7 +437,7 @@ __global__ void __launch_bounds__(NT) conv_qk_rope_bf16_kernel(
       rd[1][threadIdx.x >> 6] = sk;
     }
     // the other buffer's readers are all past their row once this is passed
-    __syncthreads();
+    lds_barrier();
     float rq = 1.f, rk = 1.f;
     {
       float a = 0.f, e = 0.f;
@@ -531,8 +543,8 @@ AF_EXPORT int afm_conv_qk_rope_cache(
   auto al = [](const void* q, size_t n) { return (uintptr_t)q % n == 0; };
   const size_t sm2 = (size_t)2 * (nq + nk) * sizeof(float);
   const int groups = (C + 3) / 4;
-  const int nt = step ? 1024 : 256, ng = (groups + nt - 1) / nt;
-  const bool fast = dt == 0 && taps <= 4 && ng <= (step ? 2 : 8) &&
+  const int nt = step ? 1024 : 512, ng = (groups + nt - 1) / nt;
+  const bool fast = dt == 0 && taps <= 4 && ng <= (step ? 2 : 4) &&
       dk % 4 == 0 && dv % 4 == 0 && ldp % 4 == 0 && rot % 8 == 0 &&
       sm2 <= 60000 && al(p, 8) && al(qo, 8) && al(cw, 8) && al(state, 8) &&
       al(qw, 8) && al(kw, 8) && al(kc, 8) && al(vc, 8) && al(tab, 16);
@@ -546,10 +558,10 @@ AF_EXPORT int afm_conv_qk_rope_cache(
 #define CQN(TP)                                                              \
   do {                                                                       \
     if (step) { if (ng <= 1) CQF(TP, 1, 1024, true); else CQF(TP, 2, 1024, true); } \
-    else if (ng <= 2) CQF(TP, 2, 256, false);                                \
-    else if (ng <= 4) CQF(TP, 4, 256, false);                                \
-    else if (ng <= 6) CQF(TP, 6, 256, false);                                \
-    else CQF(TP, 8, 256, false);                                             \
+    else if (ng <= 1) CQF(TP, 1, 512, false);                                \
+    else if (ng <= 2) CQF(TP, 2, 512, false);                                \
+    else if (ng <= 3) CQF(TP, 3, 512, false);                                \
+    else CQF(TP, 4, 512, false);                                             \
   } while (0)
     if (taps == 1) CQN(1);
     else if (taps == 2) CQN(2);

@@ -333,7 +333,9 @@ class SadupelLayer(nn.Module):
         if ff:
             sm.relu2(p[:, self.u0:self.u0 + ff], out=act[:, no:],
                      row_weight=wd if static else None, unit=f.ff, lead=ns)
-        a = sm.matmul(act, self.w_out[:, :no + ff])
+        a = sm.split_k_parts(act, self.w_out) if not md.is_prefill else None
+        if a is None:
+            a = sm.matmul(act, self.w_out[:, :no + ff])
         if f is not None and not static:
             ys, pos = self.mlp.run_sorted(h, idx, self.w_in[self.u0 + ns:],
                                           self.w_out[:, no + ns:])

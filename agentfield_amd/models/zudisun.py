@@ -358,10 +358,9 @@ class RoutedExperts(nn.Module):
     def route(self, h, dense: bool):
         """(chosen experts [T, top], their weights, dense weights or None)."""
         s = self.spec
-        z = sm.matmul(h.float(), self.router)
-        return sm.moe_route(z, self.correction, s.top, s.groups, s.keep,
-                            s.scale, dense=dense, score=s.score,
-                            renorm=s.renorm, group_top=s.group_top)
+        return sm.moe_router(h, self.router, self.correction, s.top, s.groups,
+                             s.keep, s.scale, dense=dense, score=s.score,
+                             renorm=s.renorm, group_top=s.group_top)
 
     def run_sorted(self, h, idx, up, down):
         """Each expert on the rows that chose it: up [E*unit, W], down [W,

@@ -135,8 +135,8 @@ def _mix_sigs() -> dict:
             "afm_scatter_state": [p, p, p, p, i, i, p],
             "afm_norm_rows": [p, p, p, p, f, i, i, i, i, i, p],
             "afm_sandwich_norm": [p, p, p, i64, i, p, p, f, f, i, i, i, p],
-            "afm_residual_norm": [p, p, p, i64, p, p, p, i, p, p, i64, i, f,
-                                  p, p, f, i, i, i, p],
+            "afm_residual_norm": [p, p, p, i64, p, i, p, p, p, i, p, p, i64,
+                                  i, f, p, p, f, i, i, i, p],
             "afm_relu2": [p, i64, p, i64, p, i64, i, i, i, i, i, p],
             "afm_xielu": [p, p, i64, p, i, i, i, p],
             "afm_headnorm_gate": [p, p, p, p, f, i, i, i, i64, i, i, p],
@@ -149,6 +149,8 @@ def _mix_sigs() -> dict:
             "afm_glu": [p, i64, i64, p, p, i64, i64, i, p, p, p, i64, i, i,
                         f, i, p],
             "afm_moe_route": [p, p, p, p, p, i, i, i, i, i, f, i, i, i, p],
+            "afm_moe_router": [p, p, p, p, i64, p, p, i, i, i, i, i, i, f, i,
+                               i, i, p],
             "afm_moe_combine": [p, p, p, p, p, p, p, i64, i, i, i, i, i, p],
         },
         "seq": {
@@ -208,6 +210,9 @@ def _mix_sigs() -> dict:
             "afm_conv_qk_rope_cache": [p, p, i64, p, i, p, p, p, p, p, p, p,
                                        p, i, p, p, p, f, i, i, i, i, i, i, i,
                                        i, p],
+        },
+        "skinny": {
+            "af_gemm_skinny_parts": [p, p, p, i, i, i, i, i, p],
         },
         "rglru": {
             "afm_rglru_gates": [p, p, p, p, p, p, p, i, i, i, i, p],

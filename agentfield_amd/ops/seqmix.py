@@ -692,6 +692,34 @@ def matmul(x: torch.Tensor, w: torch.Tensor, skinny: bool = True,
     return x @ w.t()
 
 
+# few rows against a weight whose inner dimension is the long one: from this
+# inner dimension on the split-K kernel streams the weight about twice as fast
+# as the vendor GEMM (42 against 93 us for 64 rows of 36864 -> 2048)
+SPLIT_K_MIN = 8192
+
+
+def split_k_parts(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor | None:
+    """x [M, K] @ w [N, K]^T as fp32 partial sums [parts, M, N] over pieces of
+    K, for a consumer that adds them up (residual_norm); None where the vendor
+    GEMM is the better choice."""
+    M, K = x.shape
+    N = w.shape[0]
+    if not (_gpu(x) and x.dtype == torch.bfloat16 and M <= 128
+            and K >= SPLIT_K_MIN and N <= 8192 and N % 64 == 0
+            and K % 64 == 0 and x.is_contiguous() and w.is_contiguous()):
+        return None
+    # about 512 workgroups
+    sk = max(1, min(32, 512 // (N // 64), K // 1024))
+    per = -(-K // sk)
+    per += (-per) % 64
+    sk = -(-K // per)
+    parts = torch.empty(sk, M, N, dtype=torch.float32, device=x.device)
+    rc = _L().af_gemm_skinny_parts(_lib.ptr(parts), _lib.ptr(x), _lib.ptr(w),
+                                   M, N, K, sk, per, _lib.cur_stream())
+    _lib.check(rc, "af_gemm_skinny_parts")
+    return parts
+
+
 # =====================================================================
 # Ops of post-norm hybrid decoders: sublayers read the residual itself, a
 # norm sits on each sublayer's output; selective state-space mixer, sigmoid
@@ -835,6 +863,34 @@ def moe_route(z: torch.Tensor, correction: torch.Tensor | None, top: int,
     return idx, w, wd
 
 
+def moe_router(h: torch.Tensor, router: torch.Tensor,
+               correction: torch.Tensor | None, top: int, n_groups: int = 0,
+               keep: int = 0, scale: float = 1.0, dense: bool = False,
+               score: str = "sigmoid", renorm: bool = True,
+               group_top: int = 2):
+    """moe_route of the logits router [E, W] fp32 . h: fp32 products and sums
+    whatever h's storage dtype."""
+    T, W = h.shape
+    E = router.shape[0]
+    if _gpu(h) and h.dtype == torch.bfloat16:
+        idx = torch.empty(T, top, dtype=torch.int32, device=h.device)
+        w = torch.empty(T, top, dtype=torch.float32, device=h.device)
+        wd = torch.empty(T, E, dtype=torch.float32, device=h.device) \
+            if dense else None
+        rc = _L().afm_moe_router(
+            _lib.ptr(idx), _lib.ptr(w), _lib.ptr(wd), _lib.ptr(h),
+            _rowstride(h), _lib.ptr(router), _lib.ptr(correction), T, W, E,
+            top, int(n_groups), int(keep), float(scale),
+            1 if score == "softmax" else 0, 1 if renorm else 0,
+            int(group_top), _lib.cur_stream())
+        if rc != 9004:          # 9004: sizes the fused form does not take
+            _lib.check(rc, "afm_moe_router")
+            return idx, w, wd
+    return moe_route(matmul(h.float(), router), correction, top, n_groups,
+                     keep, scale, dense=dense, score=score, renorm=renorm,
+                     group_top=group_top)
+
+
 def _expert_sum(T: int, W: int, ys, pos, weights, hin, idw) -> torch.Tensor:
     """CPU form of what the combining kernels add up: sum_r weights[t, r] *
     ys[pos[t*top + r]] (pos < 0: nothing) + (sum_i idw[t, i]) hin[t], fp32."""
@@ -888,14 +944,19 @@ def residual_norm(x: torch.Tensor, a: torch.Tensor | None, mult: float,
                   hin: torch.Tensor | None = None,
                   idw: torch.Tensor | None = None) -> torch.Tensor | None:
     """In place on the fp32 residual: x += mult * u (+ vec), u the sum of a
-    [T, W] (or None) and of the expert terms of moe_combine; with w the next
-    input x / sqrt(mean(x^2) + eps) * w is returned in `dtype`.  vec [W] fp32 is
-    not scaled."""
+    [T, W] (or None; or split_k_parts' partial sums [parts, T, W] fp32) and of
+    the expert terms of moe_combine; with w the next input x / sqrt(mean(x^2) +
+    eps) * w is returned in `dtype`.  vec [W] fp32 is not scaled."""
     T, W = x.shape
+    parts = None
+    if a is not None and a.dim() == 3:
+        a, parts = None, a
     if not _gpu(x):
         u = _expert_sum(T, W, ys, pos, weights, hin, idw)
         if a is not None:
             u += a.float()
+        if parts is not None:
+            u += parts.sum(0)
         x += mult * u
         if vec is not None:
             x += vec
@@ -907,9 +968,11 @@ def residual_norm(x: torch.Tensor, a: torch.Tensor | None, mult: float,
         if w is not None else None
     rc = _L().afm_residual_norm(
         _lib.ptr(x), _lib.ptr(h), _lib.ptr(a),
-        _rowstride(a) if a is not None else 0, _lib.ptr(ys), _lib.ptr(pos),
-        _lib.ptr(weights), weights.shape[1] if ys is not None else 0,
-        _lib.ptr(hin), _lib.ptr(idw), idw.stride(0) if idw is not None else 0,
+        _rowstride(a) if a is not None else 0, _lib.ptr(parts),
+        parts.shape[0] if parts is not None else 0, _lib.ptr(ys),
+        _lib.ptr(pos), _lib.ptr(weights),
+        weights.shape[1] if ys is not None else 0, _lib.ptr(hin),
+        _lib.ptr(idw), idw.stride(0) if idw is not None else 0,
         idw.shape[1] if idw is not None else 0, float(mult), _lib.ptr(vec),
         _lib.ptr(w), float(eps), T, W, _DT[dtype], _lib.cur_stream())
     _lib.check(rc, "afm_residual_norm")

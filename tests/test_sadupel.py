@@ -226,7 +226,7 @@ PORTIONS = ((0, 11), (11, 13), (13, 14), (14, 15), (15, 31), (31, 33),
 def test_kernel_groups_present(device):
     if device == "cuda":
         from agentfield_amd.ops import _lib
-        for group in ("glue", "seq", "conv", "rope"):
+        for group in ("glue", "seq", "conv", "rope", "skinny"):
             assert _lib.mixgroup(group) is not None  # no eager fallback
 
 
@@ -339,6 +339,34 @@ def test_residual_norm_many_rows(device):
     assert rel_err(h, orc.rms_norm(full, w, 1e-6)) < 2e-6
 
 
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("M", [1, 5, 64, 100, 128, 129])
+@pytest.mark.parametrize("N,K", [(128, 8192), (64, 9024), (2048, 33216),
+                                 (192, 8200)])
+def test_split_products_into_the_residual(device, M, N, K):
+    """Partial sums over pieces of a long inner dimension, added up by the
+    residual step; None where the other product serves."""
+    torch.manual_seed(K)
+    x = (torch.randn(M, K) * 0.1).to(torch.bfloat16).to(device)
+    w = (torch.randn(N, K) * 0.1).to(torch.bfloat16).to(device)
+    parts = sm.split_k_parts(x, w)
+    fits = device == "cuda" and M <= 128 and K % 64 == 0
+    assert (parts is not None) == fits
+    if not fits:        # any partition adds up
+        parts = torch.stack([x[:, :K // 8 * 3].float() @
+                             w[:, :K // 8 * 3].float().t(),
+                             x[:, K // 8 * 3:].float() @
+                             w[:, K // 8 * 3:].float().t()])
+    want = x.cpu().to(F64) @ w.cpu().to(F64).t()
+    x0 = torch.randn(M, N)
+    xr = x0.clone().to(device)
+    nw = 1 + 0.1 * torch.randn(N)
+    h = sm.residual_norm(xr, parts, 0.25, nw.to(device), 1e-6, torch.float32)
+    full = x0.to(F64) + 0.25 * want
+    assert rel_err(xr, full) < 2e-5
+    assert rel_err(h, orc.rms_norm(full, nw, 1e-6)) < 2e-5
+
+
 # ------------------------------------------------------------ feed-forward
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -403,6 +431,38 @@ def test_router(device, shift, r):
                               rtol=2e-6)
         dense[t, e] = torch.tensor(w, dtype=F64)
     assert torch.allclose(wd.cpu().to(F64), dense, atol=1e-6)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T", [1, 37])
+@pytest.mark.parametrize("W", [24, 200, 1032, 30])
+@pytest.mark.parametrize("r", ROUTERS[:5] + [
+    dict(experts=40, top=3), dict(experts=96, top=5, identity=12)])
+def test_router_from_rows(device, dtype, T, W, r):
+    """Logits and routing in one step: fp32 products of rows in either dtype
+    with router weights that use all their bits; strided rows."""
+    n = r["experts"] + r.get("identity", 0)
+    torch.manual_seed(n + W)
+    h = torch.randn(T, W + 8).to(dtype)
+    router = torch.randn(n, W) * 2 * W ** -0.5
+    corr = torch.randn(n) * 0.1
+    s = _spec(r, 8)
+    idx, wts, wd = sm.moe_router(
+        h.to(device)[:, :W], router.to(device), corr.to(device), s.top,
+        s.groups, s.keep, dense=True, score="softmax", renorm=False,
+        group_top=1)
+    z = h[:, :W].to(F64) @ router.to(F64).t()
+    full = torch.softmax(z, -1)
+    for t in range(T):
+        e, w = orc.choose(z[t], corr, r)
+        got = idx[t].tolist()
+        c = full[t] + corr.to(F64)
+        assert all(abs(float(c[a] - c[b])) < 1e-5 for a, b in zip(got, e))
+        assert torch.allclose(wts[t].cpu().to(F64), full[t, got], rtol=1e-5)
+        row = torch.zeros(n)
+        row[got] = wts[t].cpu()
+        assert torch.equal(wd[t].cpu(), row)
 
 
 def test_group_score_is_the_largest_not_a_sum():
@@ -495,9 +555,9 @@ GEOMS = [  # heads, kv_heads, dim, vdim, taps, rotated dims
     (4, 2, 16, 8, 3, 8), (2, 2, 8, 8, 1, 8), (6, 3, 12, 20, 4, 8),
     (4, 4, 70, 24, 2, 6), (3, 1, 5, 3, 6, 4), (6, 2, 32, 16, 2, 0),
     (1, 1, 4, 4, 4, 0), (9, 3, 7, 9, 3, 2),
-    # register tiles of 2, 4, 6 and 8 groups a thread
+    # register tiles of 1, 2, 3 and 4 groups a thread
     (8, 2, 96, 64, 3, 96), (16, 8, 128, 128, 4, 64), (32, 8, 128, 128, 4, 128),
-    (32, 12, 128, 128, 2, 128),
+    (32, 12, 128, 128, 2, 128), (32, 12, 128, 128, 1, 8),
     # rows wider than the register tiles; rows that do not fit in LDS
     (40, 20, 128, 128, 3, 32), (128, 4, 128, 8, 2, 64)]
 
