@@ -56,5 +56,5 @@ __device__ __forceinline__ float attn_dist_bias(float r1, float r2, int dist) {
 // weights afterwards: tanh(x) = 1 - 2 / (1 + e^(2x))
 __device__ __forceinline__ float attn_softcap_fast(float s, float inv_cap, float cap) {
   const float e = __expf(2.0f * s * inv_cap);
-  return cap - 2.0f * cap * __frcp_rn(1.0f + e);
+  return cap - 2.0f * cap * __builtin_amdgcn_rcpf(1.0f + e);
 }

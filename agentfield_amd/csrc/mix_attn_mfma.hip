@@ -117,17 +117,19 @@ struct DiffTail {
   float lam, diff, eps;
 };
 
-// LITE: no chunk, soft cap, distance bias or kept keys (window and sink
-// stay): what those terms keep alive costs the wide instances registers.
+// LITE 1: no chunk, soft cap, distance bias or kept keys (window and sink
+// stay): what those terms keep alive costs the wide instances registers.  LITE
+// 2: every earlier key, no distance bias (cap and sink stay): a wave compares
+// positions only in the tiles that reach past its first row.
 template <int DKC, int DVT, bool VEC, int NH, int KT, bool DIFF = false,
-          bool LITE = false>
+          int LITE = 0>
 __device__ __forceinline__ void attn_prefill_mfma_body(
     u16* __restrict__ out, const u16* __restrict__ q,
     const u16* __restrict__ kc, const u16* __restrict__ vc,
     const i32* __restrict__ bt, const i32* __restrict__ cu,
     const i32* __restrict__ q_start, const i32* __restrict__ tile_seq,
     const i32* __restrict__ tile_q0, float scale, int H, int G, int dk, int dv,
-    int page, int maxp, int chunk_in, int window, i64 ldq, const AttnExtra& ex,
+    int page, int maxp, int chunk_in, int window_in, i64 ldq, const AttnExtra& ex,
     const DiffTail& df = DiffTail{}) {
   constexpr int KS = DKC * 32 + 8;   // K row stride in LDS (elements)
   constexpr int VS = KT + 8;         // V^T / P row stride (KT tokens + pad)
@@ -135,7 +137,8 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
   constexpr int NHF = KT / 32;       // 32-key halves of P V
   constexpr int NK = DIFF ? 2 : 1;
   const int chunk = LITE ? 0 : chunk_in, first = LITE ? 0 : ex.first;
-  const bool biased = !LITE && ex.r1, capped = !LITE && ex.cap > 0.f;
+  const int window = LITE == 2 ? 0 : window_in;
+  const bool biased = !LITE && ex.r1, capped = LITE != 1 && ex.cap > 0.f;
   constexpr int XS = DVT * 16 + 4;   // row stride of the maps' exchange (floats)
   constexpr size_t KVB = sizeof(u16) * (NK * KT * KS + DVT * 16 * VS);
   constexpr size_t XB = DIFF ? sizeof(float) * 64 * XS : 0;
@@ -237,6 +240,7 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
       }
     }
     // ---- mask + online softmax; reg r is row (lane>>4)*4 + r ----
+    const bool all_seen = LITE == 2 && kv0 + KT - 1 <= wp0;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int p = wp0 + (lane >> 4) * 4 + r;
@@ -251,7 +255,8 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
         float sv = s_acc[st][r] * scale;
         if (capped) sv = attn_softcap_fast(sv, inv_cap, ex.cap);
         if (biased) sv -= bias_lds[hsel * 128 + (p - p0) - (j - kv0) + KT - 1];
-        sr[st] = (j <= p && (j >= rlo || j < first)) ? sv : AF_NEG_INF;
+        sr[st] = (all_seen || (j <= p && (LITE == 2 || j >= rlo || j < first)))
+                     ? sv : AF_NEG_INF;
         tmax = fmaxf(tmax, sr[st]);
       }
       tmax = group16_max_f32(tmax);
@@ -362,7 +367,7 @@ __device__ __forceinline__ void attn_prefill_mfma_body(
     out, q, kc, vc, bt, cu, q_start, tile_seq, tile_q0, scale, H, G, dk, dv,   \
     page, maxp, chunk, window, ldq, ex
 
-template <int DKC, int DVT, bool VEC, int NH, int KT = 64, bool LITE = false>
+template <int DKC, int DVT, bool VEC, int NH, int KT = 64, int LITE = 0>
 __global__ void __launch_bounds__(256 * NH) attn_prefill_mfma_kernel(AF_APM_PARAMS) {
   attn_prefill_mfma_body<DKC, DVT, VEC, NH, KT, false, LITE>(AF_APM_ARGS);
 }
@@ -370,7 +375,7 @@ __global__ void __launch_bounds__(256 * NH) attn_prefill_mfma_kernel(AF_APM_PARA
 // The widest instance keeps 16 x 512 output accumulators and an 18-fragment
 // query per wave: two waves per SIMD (the eight waves of one workgroup) is all
 // a CU can hold of it, so it may use their full register share.
-template <bool LITE>
+template <int LITE>
 __global__ void __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(2, 2)))
 attn_prefill_mfma_wide_pair_kernel(AF_APM_PARAMS) {
   attn_prefill_mfma_body<18, 32, true, 2, 32, false, LITE>(AF_APM_ARGS);
@@ -379,7 +384,7 @@ attn_prefill_mfma_wide_pair_kernel(AF_APM_PARAMS) {
 template <int DKC, int DVT, bool VEC, int KT = 64>
 __global__ void __launch_bounds__(512) diff_prefill_mfma_kernel(AF_APM_PARAMS,
                                                                 DiffTail df) {
-  attn_prefill_mfma_body<DKC, DVT, VEC, 2, KT, true, true>(AF_APM_ARGS, df);
+  attn_prefill_mfma_body<DKC, DVT, VEC, 2, KT, true, 1>(AF_APM_ARGS, df);
 }
 
 // ------------------------------------------------ single rows, many heads
@@ -633,7 +638,8 @@ AF_EXPORT int afm_attn_prefill_mfma(
                      cap, ldv, keep_first, vshare, gate, ldg, ldo};
   // two heads per workgroup when a K/V group has an even number of them
   const bool pair = vec && (H / G) % 2 == 0;
-  const bool lite = chunk <= 0 && cap <= 0.f && !r1 && keep_first == 0;
+  const bool plain = chunk <= 0 && !r1 && keep_first == 0;
+  const bool lite = plain && cap <= 0.f, causal = plain && window <= 0;
   hipStream_t s = (hipStream_t)stream;
 #define APM(DKC, DVT, VEC, NH, ...)                                            \
   attn_prefill_mfma_kernel<DKC, DVT, VEC, NH, ##__VA_ARGS__>                   \
@@ -652,16 +658,17 @@ AF_EXPORT int afm_attn_prefill_mfma(
       (const i32*)bt, (const i32*)cu, (const i32*)q_start,                     \
       (const i32*)tile_seq, (const i32*)tile_q0, scale, H, G, dk, dv, page,    \
       maxp, chunk, window, ldq, ex)
-    if (pair && lite) APW(true);
-    else if (pair) APW(false);
+    if (pair && lite) APW(1);
+    else if (pair) APW(0);
 #undef APW
     else
       APM(18, 32, true, 1);
   }
-  else if (dk > 128 || dv > 128) { if (pair && lite) APM(10, 16, true, 2, 64, true); else if (pair) APM(10, 16, true, 2); else APM(10, 16, true, 1); }
+  else if (dk > 128 || dv > 128) { if (pair && lite) APM(10, 16, true, 2, 64, 1); else if (pair) APM(10, 16, true, 2); else APM(10, 16, true, 1); }
   else if (small && pair) APM(2, 4, true, 2);
   else if (small && vec) APM(2, 4, true, 1);
   else if (small) APM(2, 4, false, 1);
+  else if (pair && causal) APM(4, 8, true, 2, 64, 2);
   else if (pair) APM(4, 8, true, 2);
   else if (vec) APM(4, 8, true, 1);
   else APM(4, 8, false, 1);

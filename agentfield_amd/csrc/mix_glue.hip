@@ -893,7 +893,7 @@ __global__ void __launch_bounds__(NW * 64) moe_router_kernel(
   f32x4 acc[ET];
 #pragma unroll
   for (int et = 0; et < ET; ++et) acc[et] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
+#pragma unroll 4
   for (int k0 = wid * 32; k0 < W; k0 += NW * 32) {
     const int k = k0 + (lane >> 4) * 8;    // W is a multiple of 8
     union { s16x8 s; bf16x8 b; } a;

@@ -322,22 +322,24 @@ class SadupelLayer(nn.Module):
         terms: dict = {}
         static = f is not None and self.mlp.is_static(T, md)
         ff = ns + (self.n_experts if static else 0)     # units run on all rows
-        p = sm.matmul(h, self.w_in[:self.u0 + ff])
-        act = torch.empty(T, no + ff, dtype=h.dtype, device=h.device)
-        self.mixer(p, cache, run, md, positions, ctx, act[:, :no])
-        wd = None
+        wd = plan = None
         if f is not None:
             idx, wts, wd = self.mlp.route(h, static or f.identity > 0)
             if f.identity:
                 terms.update(hin=h, idw=wd[:, f.experts:])
+            if not static:
+                plan = self.mlp.sort(idx)
+        p = sm.matmul(h, self.w_in[:self.u0 + ff])
+        act = torch.empty(T, no + ff, dtype=h.dtype, device=h.device)
+        self.mixer(p, cache, run, md, positions, ctx, act[:, :no])
         if ff:
             sm.relu2(p[:, self.u0:self.u0 + ff], out=act[:, no:],
                      row_weight=wd if static else None, unit=f.ff, lead=ns)
         a = sm.split_k_parts(act, self.w_out) if not md.is_prefill else None
         if a is None:
             a = sm.matmul(act, self.w_out[:, :no + ff])
-        if f is not None and not static:
-            ys, pos = self.mlp.run_sorted(h, idx, self.w_in[self.u0 + ns:],
+        if plan is not None:
+            ys, pos = self.mlp.run_sorted(h, plan, self.w_in[self.u0 + ns:],
                                           self.w_out[:, no + ns:])
             if ys is not None:
                 terms.update(ys=ys, pos=pos, weights=wts)

@@ -362,22 +362,40 @@ class RoutedExperts(nn.Module):
                              s.keep, s.scale, dense=dense, score=s.score,
                              renorm=s.renorm, group_top=s.group_top)
 
-    def run_sorted(self, h, idx, up, down):
+    def sort(self, idx):
+        """(row, choice) pairs in expert order, for run_sorted.  Their counts
+        start on the way to the host here, so that what is queued between the
+        two calls runs while the host waits for them."""
+        s = self.spec
+        flat = idx.flatten().long()
+        order = torch.argsort(flat, stable=True)
+        counts = torch.bincount(flat, minlength=s.experts + s.identity)
+        ready = None
+        if counts.is_cuda:
+            host = torch.empty(counts.shape, dtype=counts.dtype,
+                               pin_memory=True)
+            host.copy_(counts, non_blocking=True)
+            ready = torch.cuda.Event()
+            ready.record()
+            counts = host
+        pos = torch.empty_like(order, dtype=torch.int32)
+        pos[order] = torch.arange(order.numel(), dtype=torch.int32,
+                                  device=idx.device)
+        if s.identity:
+            pos.masked_fill_(flat >= s.experts, -1)
+        return order, pos, counts, ready
+
+    def run_sorted(self, h, plan, up, down):
         """Each expert on the rows that chose it: up [E*unit, W], down [W,
         E*F].  Returns (expert outputs in expert order, None without any; the
         place of every (row, choice) in them, -1 for identity experts)."""
         s = self.spec
         E, F, U = s.experts, s.ff, s.unit
-        # (row, choice) pairs in expert order; one host round trip for sizes
-        flat = idx.flatten().long()
-        order = torch.argsort(flat, stable=True)
-        counts = torch.bincount(flat, minlength=E + s.identity).tolist()[:E]
-        pos = torch.empty_like(order, dtype=torch.int32)
-        pos[order] = torch.arange(order.numel(), dtype=torch.int32,
-                                  device=h.device)
+        order, pos, counts, ready = plan
+        if ready is not None:
+            ready.synchronize()
+        counts = counts.tolist()[:E]
         n = sum(counts)
-        if s.identity:
-            pos.masked_fill_(flat >= E, -1)
         if n == 0:
             return None, pos
         xs = h.index_select(0, torch.div(order[:n], s.top,
@@ -411,7 +429,8 @@ class RoutedExperts(nn.Module):
                 sm.glu(gu[:, E * 2 * F:], Fs, s.act, out=act[:, E * F:],
                        limit=s.limit)
             return sm.matmul(act, self.down), None
-        ys, pos = self.run_sorted(h, idx, self.gate_up, self.down)
+        plan = self.sort(idx)
+        ys, pos = self.run_sorted(h, plan, self.gate_up, self.down)
         shared = None
         if Fs > 0:
             a = sm.glu(sm.matmul(h, self.gate_up[E * 2 * F:]), Fs, s.act,

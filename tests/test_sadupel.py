@@ -119,7 +119,21 @@ def cfg_odd():
                        _moe(3, 2, 25, 11, None, 2))]}
 
 
-ZOO = {"mixed": cfg_mixed, "degenerate": cfg_degenerate, "odd": cfg_odd}
+def cfg_wide():
+    """Many small experts: an output product long enough for the split-K
+    kernel of decode steps, a router of 128 outputs in 16 groups."""
+    return {"architecture": "Sadupel", "vocab": 64, "width": 64,
+            "residual_mult": 0.6, "norm": {"eps": 1e-6},
+            "embedding": {"bigram": {"buckets": 29, "mul_prev": 7,
+                                     "mul_cur": 3}},
+            "layers": [
+                _layer(_attn(8, 1, 16, 32, 3, 0.3, 6.0,
+                             {"dims": 16, "base": 1000.0}),
+                       _moe(124, 4, 64, 64, (16, 5), 4))]}
+
+
+ZOO = {"mixed": cfg_mixed, "degenerate": cfg_degenerate, "odd": cfg_odd,
+       "wide": cfg_wide}
 
 
 def build(cfg_json, device, dtype, seed=0, page=8, pages=64, live=4,
@@ -499,7 +513,7 @@ def test_sorted_experts(device, dtype, T, r):
     down = torch.cat([P[n + "down"] for n in names], 1).to(device, dtype)
     hd = h.to(device)
     idx, wts, wd = mod.route(hd, True)
-    ys, pos = mod.run_sorted(hd, idx, up, down)
+    ys, pos = mod.run_sorted(hd, mod.sort(idx), up, down)
     kw = {}
     if r.get("identity"):
         kw = dict(hin=hd, idw=wd[:, r["experts"]:])
@@ -528,7 +542,8 @@ def test_only_identity_experts_chosen(device):
     h = torch.randn(20, W, device=device)
     idx, _w, wd = mod.route(h, True)
     assert idx.tolist() == [[4, 3]] * 20
-    ys, pos = mod.run_sorted(h, idx, torch.zeros(24, W, device=device),
+    ys, pos = mod.run_sorted(h, mod.sort(idx),
+                             torch.zeros(24, W, device=device),
                              torch.zeros(W, 24, device=device))
     assert ys is None and bool((pos == -1).all())
     x = torch.zeros(20, W, device=device)
@@ -919,12 +934,13 @@ def test_oracle_tells_loops_apart(change):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_greedy_generation_through_scheduler(device, dtype):
+@pytest.mark.parametrize("name", ["mixed", "wide"])
+def test_greedy_generation_through_scheduler(device, dtype, name):
     """engine.generate: the scheduler's batched prefill, (on GPU) the
     graph-captured decode step and the sampler reproduce the oracle's greedy
     continuation of unequal prompts; a second batch replays the same graphs
     over reused pages and slots."""
-    cj = cfg_mixed()
+    cj = ZOO[name]()
     eng, w = build(cj, device, dtype, paced=False,
                    graphs=(device == "cuda"), pages=48)
     # the GPU sampler reads logits rounded to bf16, so near-ties may fall
