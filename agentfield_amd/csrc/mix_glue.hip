@@ -895,22 +895,20 @@ __global__ void __launch_bounds__(NW * 64) moe_router_kernel(
   for (int et = 0; et < ET; ++et) acc[et] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
   for (int k0 = wid * 32; k0 < W; k0 += NW * 32) {
-    const int k = k0 + (lane >> 4) * 8;    // W is a multiple of 8
+    // loads without conditions, so that several steps' are in flight: past W
+    // (a multiple of 8) the h fragment is zero, columns past E are never read
+    const int k = k0 + (lane >> 4) * 8, kc = min(k, W - 8);
     union { s16x8 s; bf16x8 b; } a;
-    a.s = s16x8{0, 0, 0, 0, 0, 0, 0, 0};
-    if (k < W) a.s = *reinterpret_cast<const s16x8*>(hr + k);
+    a.s = *reinterpret_cast<const s16x8*>(hr + kc);
+    if (k >= W) a.s = s16x8{0, 0, 0, 0, 0, 0, 0, 0};
 #pragma unroll
     for (int et = 0; et < ET; ++et) {
-      const int n = et * 16 + (lane & 15);
+      const int n = min(et * 16 + (lane & 15), E - 1);
+      const f32x4* rp = reinterpret_cast<const f32x4*>(router + (size_t)n * W + kc);
+      const f32x4 r0 = rp[0], r1 = rp[1];
       float r[8];
 #pragma unroll
-      for (int j = 0; j < 8; ++j) r[j] = 0.f;
-      if (n < E && k < W) {
-        const f32x4* rp = reinterpret_cast<const f32x4*>(router + (size_t)n * W + k);
-        const f32x4 r0 = rp[0], r1 = rp[1];
-#pragma unroll
-        for (int j = 0; j < 4; ++j) { r[j] = r0[j]; r[4 + j] = r1[j]; }
-      }
+      for (int j = 0; j < 4; ++j) { r[j] = r0[j]; r[4 + j] = r1[j]; }
 #pragma unroll
       for (int term = 0; term < 3; ++term) {
         bf16x8 b;
