@@ -81,7 +81,7 @@ def parse_args():
                    help="instead of the default workload: engine-level "
                         "prefill and decode token throughput of the hybrid "
                         "families (Reperax, Zudisun, Fugevik, Vabedra, "
-                        "Fironex) beside each other and "
+                        "Fironex, Sadupel) beside each other and "
                         "the Llama family at equal width / ff / depth, "
                         "random weights; one JSON line per model and phase "
                         "(single GPU)")
